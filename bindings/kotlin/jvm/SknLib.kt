@@ -14,7 +14,7 @@ import java.lang.foreign.ValueLayout.JAVA_LONG
 import java.lang.invoke.MethodHandle
 
 object SknLib {
-    const val ABI_VERSION = 3
+    const val ABI_VERSION = 4
     const val OK = 0
     const val ERR_ARG = -1
     const val ERR_TYPE = -2
@@ -84,6 +84,21 @@ object SknLib {
     val llamaPrefill: MethodHandle = h("skn_llama_prefill", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, ADDRESS, JAVA_INT, ADDRESS))
     val llamaDecode: MethodHandle = h("skn_llama_decode", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_INT, JAVA_INT, ADDRESS))
     val llamaLogits: MethodHandle = h("skn_llama_logits", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, ADDRESS))
+    val kvCreateShared: MethodHandle = h("skn_kv_create_shared", FunctionDescriptor.of(JAVA_INT, ADDRESS, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, ADDRESS))
+    val attnShared: MethodHandle = h("skn_attn_shared", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_INT, ADDRESS, ADDRESS, ADDRESS, JAVA_INT, ADDRESS))
+    val rstateCreate: MethodHandle = h("skn_rstate_create", FunctionDescriptor.of(JAVA_INT, ADDRESS, JAVA_INT, JAVA_INT, JAVA_INT, ADDRESS))
+    val rstateFree: MethodHandle = h("skn_rstate_free", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS))
+    val rstateReset: MethodHandle = h("skn_rstate_reset", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_INT))
+    val deltaRule: MethodHandle = h("skn_delta_rule", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_INT, ADDRESS, ADDRESS, ADDRESS, ADDRESS, ADDRESS, JAVA_INT, ADDRESS))
+    val rmsnormGrouped: MethodHandle = h("skn_rmsnorm_grouped", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, ADDRESS, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_FLOAT, ADDRESS))
+    val xielu: MethodHandle = h("skn_xielu", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_LONG, JAVA_FLOAT, JAVA_FLOAT, ADDRESS))
+    val hybridCreate: MethodHandle = h("skn_hybrid_create", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, ADDRESS, ADDRESS))
+    val hybridFree: MethodHandle = h("skn_hybrid_free", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS))
+    val hybridReset: MethodHandle = h("skn_hybrid_reset", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS))
+    val hybridPrefill: MethodHandle = h("skn_hybrid_prefill", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, ADDRESS, JAVA_INT, ADDRESS))
+    val hybridDecode: MethodHandle = h("skn_hybrid_decode", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_INT, JAVA_INT, ADDRESS))
+    val hybridExtend: MethodHandle = h("skn_hybrid_extend", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, ADDRESS, JAVA_INT, ADDRESS, JAVA_INT, ADDRESS))
+    val hybridLogits: MethodHandle = h("skn_hybrid_logits", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, ADDRESS))
     val synthWeight: MethodHandle = h("skn_synth_weight", FunctionDescriptor.of(JAVA_INT, JAVA_INT, JAVA_LONG, JAVA_LONG, JAVA_LONG, ADDRESS, JAVA_LONG))
     val synthActivationF32: MethodHandle = h("skn_synth_activation_f32", FunctionDescriptor.of(JAVA_INT, JAVA_LONG, JAVA_LONG, ADDRESS))
     val synthActivationBf16: MethodHandle = h("skn_synth_activation_bf16", FunctionDescriptor.of(JAVA_INT, JAVA_LONG, JAVA_LONG, ADDRESS))

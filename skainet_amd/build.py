@@ -1,11 +1,13 @@
 """Builds libskainet_hip.so (hand-written HIP for gfx950) in-tree with hipcc.
 
     python -m skainet_amd.build            # compile every csrc/*.hip and link skainet_amd/libskainet_hip.so
+    python -m skainet_amd.build --dense    # only what models with dense weights need: skainet_amd/libskainet_dense.so
 
 hipcc cross-compiles for gfx950 without a GPU.  The library has no dependency beyond the HIP runtime.
 """
 from __future__ import annotations
 
+import fcntl
 import glob
 import os
 import shutil
@@ -17,6 +19,10 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 OBJ = os.path.join(CSRC, "build")
 LIB = os.path.join(HERE, "libskainet_hip.so")
+DENSE_LIB = os.path.join(HERE, "libskainet_dense.so")
+# the sources of the layer-list decoder over bf16 / fp32 weights and of nothing else (seconds to compile; the
+# block-quantized matvecs alone take minutes)
+DENSE_SOURCES = ("api", "kvcache", "stepper", "dense_gemm", "dense_matvec", "dense_rows", "attention_prefill", "attention_shared", "delta", "hybrid")
 
 ARCH = "gfx950"
 # packed-fp32 VALU forms are kept off: scalar fp32 code must not be fused into v_pk_* instructions
@@ -41,9 +47,11 @@ def _run(cmd):
     return out
 
 
-def build_library(jobs=8, verbose=False, save_temps=False):
+def build_library(jobs=8, verbose=False, save_temps=False, dense_only=False):
     os.makedirs(OBJ, exist_ok=True)
     sources = sorted(glob.glob(os.path.join(CSRC, "*.hip")))
+    if dense_only:
+        sources = [os.path.join(CSRC, f"{n}.hip") for n in DENSE_SOURCES]
     if not sources:
         raise RuntimeError("no HIP sources found")
     objs = [os.path.join(OBJ, os.path.basename(s)[:-4] + ".o") for s in sources]
@@ -57,9 +65,23 @@ def build_library(jobs=8, verbose=False, save_temps=False):
         for src, out in zip(sources, ex.map(compile_one, zip(sources, objs))):
             if verbose and out.strip():
                 print(f"--- {os.path.basename(src)}\n{out}")
-    _run([hipcc(), f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", LIB, *objs])
-    return LIB
+    lib = DENSE_LIB if dense_only else LIB
+    # linked beside its place and moved there: no process ever loads a half-written library
+    _run([hipcc(), f"--offload-arch={ARCH}", "-shared", "-fPIC", "-Wl,--no-undefined", "-o", lib + ".new", *objs])
+    os.replace(lib + ".new", lib)
+    return lib
+
+
+def ensure_library():
+    """For programs that run a dense model from a fresh checkout: compiles the dense part unless a library is there."""
+    if os.path.exists(LIB) or os.path.exists(DENSE_LIB):
+        return
+    os.makedirs(OBJ, exist_ok=True)
+    with open(os.path.join(OBJ, "lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)  # (two programs started at once: the second finds the first one's library)
+        if not os.path.exists(DENSE_LIB):
+            build_library(dense_only=True)
 
 
 if __name__ == "__main__":
-    print(build_library(verbose=True, save_temps="--save-temps" in sys.argv))
+    print(build_library(verbose=True, save_temps="--save-temps" in sys.argv, dense_only="--dense" in sys.argv))

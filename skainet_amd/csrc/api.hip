@@ -3,6 +3,12 @@
 
 static thread_local std::string g_ctxless_error;
 
+static std::vector<int (*)(skn_ctx*)>& family_inits() {
+    static std::vector<int (*)(skn_ctx*)> inits;
+    return inits;
+}
+skn_family::skn_family(int (*init)(skn_ctx* ctx)) { family_inits().push_back(init); }
+
 int skn_fail(skn_ctx* ctx, int code, const char* fmt, ...) {
     char buf[512];
     va_list ap;
@@ -71,9 +77,9 @@ int skn_init(int device, skn_ctx** out) {
         ctx->profiler_attached = (tool && *tool) || (pre && strstr(pre, "rocprofiler"));
         if (ctx->profiler_attached) ctx->opt_llama_graph = 0;
     }
-    int rc = skn_matvec_init(ctx);
-    if (rc == SKN_OK) rc = skn_gemm_init(ctx);
-    if (rc == SKN_OK) rc = skn_attn_init(ctx);
+    int rc = SKN_OK;
+    for (auto init : family_inits())
+        if (rc == SKN_OK) rc = init(ctx);
     if (rc != SKN_OK) {
         g_ctxless_error = ctx->err;
         skn_shutdown(ctx);
@@ -283,6 +289,7 @@ int skn_set_option(skn_ctx* ctx, const char* key, int value) {
     else if (!strcmp(key, "llama.fused")) ctx->opt_llama_fused = value;
     else if (!strcmp(key, "llama.expand_weights")) ctx->opt_llama_expand = value;
     else if (!strcmp(key, "gemm.tile")) ctx->opt_gemm_tile = value;
+    else if (!strcmp(key, "dense.tile")) ctx->opt_dense_tile = value;
     else if (!strcmp(key, "gemm.q6k_fused")) ctx->opt_gemm_q6k_fused = value;
     else if (!strcmp(key, "matvec.stage")) ctx->opt_matvec_stage = value;
     else if (!strcmp(key, "test.rope_table")) ctx->opt_test_rope_table = value;

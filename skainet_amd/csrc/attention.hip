@@ -23,16 +23,6 @@ constexpr int kAttnThreads = 256;
 constexpr int kMaxSplits = 512;
 constexpr int kUnroll = 4;  // tokens per stream in flight per iteration (K and V: 8 x 16 bytes per lane)
 
-template <int LPT>
-__device__ __forceinline__ float group_sum(float v) {
-    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, true));   // lane ^ 1
-    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x4E, 0xF, 0xF, true));   // lane ^ 2
-    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x141, 0xF, 0xF, true));  // 7 - lane
-    if constexpr (LPT >= 16) v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x140, 0xF, 0xF, true));
-    if constexpr (LPT >= 32) v += __shfl_xor(v, 16, 64);
-    return v;
-}
-
 __device__ __forceinline__ float dot8(const u32x4& k, const float (&qf)[8]) {
     float s = 0.f;
 #pragma unroll
@@ -114,7 +104,7 @@ __global__ __launch_bounds__(kAttnThreads) void attn_decode_kernel(
         float m_new = m_run;
 #pragma unroll
         for (int u = 0; u < U; u++) {
-            const float d = group_sum<LPT>(dot8(kk[u], qf));
+            const float d = lane_group_sum<LPT>(dot8(kk[u], qf));
             sc[u] = ok[u] ? d : -INFINITY;
             m_new = fmaxf(m_new, sc[u]);
         }
@@ -298,7 +288,7 @@ __global__ __launch_bounds__(kWideThreads) void attn_decode_wide_kernel(
         float m_new = m_run;
 #pragma unroll
         for (int u = 0; u < U; u++) {
-            const float d = group_sum<LPT>(dot8(kk[u], qf));
+            const float d = lane_group_sum<LPT>(dot8(kk[u], qf));
             sc[u] = ok[u] ? d : -INFINITY;
             m_new = fmaxf(m_new, sc[u]);
         }
@@ -383,6 +373,7 @@ int skn_attn_launch_ex(skn_ctx* ctx, skn_kv* kv, const float* q_dev, const int32
                        int seq_fixed, int n_splits, float* partial, int* counters, float scale, float* out_dev,
                        int n_q_head) {
     const int D = kv->head_dim;
+    SKN_REQUIRE(ctx, !kv->shared, SKN_ERR_STATE, "attention: the cache shares its keys and values (skn_attn_shared reads it)");
     if (n_q_head <= 0) n_q_head = kv->n_head;
     SKN_REQUIRE(ctx, n_q_head % kv->n_head == 0, SKN_ERR_SHAPE,
                 "attention: %d query heads are not a multiple of the %d cached heads", n_q_head, kv->n_head);
@@ -417,6 +408,7 @@ int skn_attn_launch_ex(skn_ctx* ctx, skn_kv* kv, const float* q_dev, const int32
 int skn_attn_launch_unmerged(skn_ctx* ctx, skn_kv* kv, const float* q_dev, const int32_t* nctx_dev, int n_queries,
                              int seq_fixed, int n_splits, float* opart, float* ml, float scale, float* out_dev, int n_q_head) {
     const int D = kv->head_dim;
+    SKN_REQUIRE(ctx, !kv->shared, SKN_ERR_STATE, "attention: the cache shares its keys and values (skn_attn_shared reads it)");
     if (n_q_head <= 0) n_q_head = kv->n_head;
     SKN_REQUIRE(ctx, n_q_head % kv->n_head == 0, SKN_ERR_SHAPE,
                 "attention: %d query heads are not a multiple of the %d cached heads", n_q_head, kv->n_head);
@@ -489,7 +481,7 @@ __global__ void attn_clear_counters_kernel(int* counters, int n) {
 }  // namespace
 
 // Called by skn_init with the context's device current.
-int skn_attn_init(skn_ctx* ctx) {
+static int skn_attn_init(skn_ctx* ctx) {
     SKN_REQUIRE(ctx, ctx->device >= 0 && ctx->device < kMaxDevices, SKN_ERR_ARG, "device index %d is beyond %d", ctx->device,
                 kMaxDevices);
     if (!g_static_scratch[ctx->device]) {
@@ -500,6 +492,7 @@ int skn_attn_init(skn_ctx* ctx) {
     }
     return SKN_OK;
 }
+static skn_family register_family(skn_attn_init);
 
 extern "C" int skn_attn_decode_static(skn_ctx* ctx, skn_kv* kv, const float* q_dev, float scale, float* out_dev) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_attn_decode_static: ctx is null");

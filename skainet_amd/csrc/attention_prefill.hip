@@ -13,6 +13,7 @@
 // Precision: K and V are the cached fp16 values; q (pre-multiplied by scale * log2 e) and P enter as fp16 pairs
 // hi + lo (two matrix instructions per step), products and sums are fp32.
 #include "kv.h"
+#include "dense.h"
 
 namespace {
 
@@ -30,9 +31,11 @@ __device__ __forceinline__ int key_of(int s, int h, int p) { return 16 * s + 8 *
 // kfrag: [head][tile][k-step D/16][lane] x 8 halves: lane 32 h + r = elements 16 s + 8 h .. + 7 of key r.
 // vfrag: [head][tile][32-row block of d][k-step 2][lane] x 8 halves: lane 32 h + r = element 32 b + r of the
 //        eight keys key_of(s, h, 0..7).
-template <int D>
+// SHARED: a cache that shares its keys and values (kv.h): the row is the value, and times its token's key_scale the key.
+template <int D, bool SHARED>
 __global__ __launch_bounds__(256) void attn_frag_kernel(const uint16_t* __restrict__ k_pool, const uint16_t* __restrict__ v_pool,
-                                                        const int32_t* __restrict__ table, int n_head, int page_tokens,
+                                                        const float* __restrict__ key_scale, const int32_t* __restrict__ table,
+                                                        int n_head, int page_tokens,
                                                         int n_tokens, int n_tiles, u32x4* __restrict__ kfrag,
                                                         u32x4* __restrict__ vfrag) {
     constexpr int kPieces = D / 8;             // 16-byte pieces of a row
@@ -49,7 +52,16 @@ __global__ __launch_bounds__(256) void attn_frag_kernel(const uint16_t* __restri
             const int page = table[t / page_tokens], slot = t % page_tokens;
             const size_t off = (((size_t)page * n_head + head) * page_tokens + slot) * D + 8 * pc;
             kk = *reinterpret_cast<const u32x4*>(k_pool + off);
-            vv = *reinterpret_cast<const u32x4*>(v_pool + off);
+            if constexpr (SHARED) {
+                vv = kk;
+                const float f = key_scale[(size_t)page * page_tokens + slot];
+                half8_t x = __builtin_bit_cast(half8_t, kk);
+#pragma unroll
+                for (int e = 0; e < 8; e++) x[e] = (_Float16)((float)x[e] * f);
+                kk = __builtin_bit_cast(u32x4, x);
+            } else {
+                vv = *reinterpret_cast<const u32x4*>(v_pool + off);
+            }
         }
         kout[(pc >> 1) * 64 + 32 * (pc & 1) + r] = kk;
         *reinterpret_cast<u32x4*>(vt + r * kPitch + 8 * pc) = vv;
@@ -70,11 +82,16 @@ __global__ __launch_bounds__(256) void attn_frag_kernel(const uint16_t* __restri
 
 // grid (query blocks of 32, heads), four wavefronts each; the block with the most keys first.
 // q, out: fp32 [n_queries][n_head][D]; query row t attends to keys [0, first_ctx + t).
-template <int D>
+// BIAS: the scores lose slope_h * distance, slope_h = 2^(-8 (h + 1) / n_head), and the output is `dim` of D elements per
+// head in rows of ldo, fp32 or bf16.
+struct PrefillExt {
+    int dim = 0, ldo = 0, out_type = SKN_TYPE_F32;
+};
+template <int D, bool BIAS>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) void attn_prefill_kernel(const float* __restrict__ q, const u32x4* __restrict__ kfrag,
                                                           const u32x4* __restrict__ vfrag, float* __restrict__ out,
                                                           int n_queries, int n_head, int kv_group, int first_ctx, int n_tiles,
-                                                          float scale_log2e) {
+                                                          float scale_log2e, PrefillExt ext) {
     constexpr int KS = D / 16, DB = D / 32;
     __shared__ float part[3][DB * 16 + 2][64];  // running maximum, sum and accumulators of wavefronts 1..3
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, h = lane >> 5, n = lane & 31;
@@ -103,6 +120,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
     for (int b = 0; b < DB; b++)
 #pragma unroll
         for (int x = 0; x < 16; x++) o[b][x] = 0.f;
+    const float slope = BIAS ? exp2f(-8.0f * (float)(head + 1) / (float)n_head) * 1.4426950408889634f : 0.f;
     float mrun = -INFINITY, lrun = 0.f;  // running maximum (both halves agree) and this half's share of the sum
 
     // (grouped queries: kv_group consecutive query heads read the keys and values of one cached head)
@@ -134,6 +152,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
 #pragma unroll
         for (int x = 0; x < 16; x++) {
             const int key = 32 * tile + 8 * (x >> 2) + 4 * h + (x & 3);
+            if constexpr (BIAS) sc[x] = fmaf(slope, (float)(key - (n_ctx - 1)), sc[x]);
             sc[x] = key < n_ctx ? sc[x] : -INFINITY;
             mt = fmaxf(mt, sc[x]);
         }
@@ -204,7 +223,19 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
     }
     const float ltot = lrun + __shfl_xor(lrun, 32);
     const float inv = ltot > 0.f ? 1.0f / ltot : 0.f;
-    if (32 * qb + n < n_queries) {
+    if (BIAS && 32 * qb + n < n_queries) {
+#pragma unroll
+        for (int b = 0; b < DB; b++)
+#pragma unroll
+            for (int x = 0; x < 16; x++) {
+                const int d = 32 * b + 8 * (x >> 2) + 4 * h + (x & 3);
+                const size_t at = (size_t)t * ext.ldo + (size_t)head * ext.dim + d;
+                if (d >= ext.dim) continue;
+                if (ext.out_type == SKN_TYPE_F32) reinterpret_cast<float*>(out)[at] = o[b][x] * inv;
+                else reinterpret_cast<uint16_t*>(out)[at] = skn_bf16_bits(o[b][x] * inv);
+            }
+    }
+    if (!BIAS && 32 * qb + n < n_queries) {
         float* orow = out + ((size_t)t * n_head + head) * D + 4 * h;
 #pragma unroll
         for (int b = 0; b < DB; b++)
@@ -215,9 +246,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
     }
 }
 
-template <int D>
+template <int D, bool SHARED>
 int launch_prefill(skn_ctx* ctx, skn_kv* kv, int seq, const float* q_dev, int n_queries, int first_ctx, float scale,
-                   float* out_dev, int n_q_head) {
+                   float* out_dev, int n_q_head, PrefillExt ext = PrefillExt()) {
     const int n_tokens = first_ctx + n_queries - 1;  // keys the last query sees
     const int n_tiles = (n_tokens + 31) / 32;
     const size_t frag_bytes = (size_t)kv->n_head * n_tiles * 32 * D * 2;
@@ -235,13 +266,14 @@ int launch_prefill(skn_ctx* ctx, skn_kv* kv, int seq, const float* q_dev, int n_
     }
     u32x4* kfrag = (u32x4*)ctx->prefill_ws;
     u32x4* vfrag = (u32x4*)((uint8_t*)ctx->prefill_ws + frag_bytes);
-    skn_launch(ctx, attn_frag_kernel<D>, dim3(n_tiles, kv->n_head), dim3(256), 0, (const uint16_t*)kv->k_pool,
-               (const uint16_t*)kv->v_pool, (const int32_t*)(kv->page_table_dev + (size_t)seq * kv->pages_per_seq), kv->n_head,
+    skn_launch(ctx, attn_frag_kernel<D, SHARED>, dim3(n_tiles, kv->n_head), dim3(256), 0, (const uint16_t*)kv->k_pool,
+               (const uint16_t*)kv->v_pool, (const float*)kv->key_scale,
+               (const int32_t*)(kv->page_table_dev + (size_t)seq * kv->pages_per_seq), kv->n_head,
                kv->page_tokens, n_tokens, n_tiles, kfrag, vfrag);
     SKN_LAUNCH_CHECK(ctx);
-    skn_launch(ctx, attn_prefill_kernel<D>, dim3((n_queries + 31) / 32, n_q_head), dim3(256), 0, q_dev, (const u32x4*)kfrag,
+    skn_launch(ctx, attn_prefill_kernel<D, SHARED>, dim3((n_queries + 31) / 32, n_q_head), dim3(256), 0, q_dev, (const u32x4*)kfrag,
                (const u32x4*)vfrag, out_dev, n_queries, n_q_head, n_q_head / kv->n_head, first_ctx, n_tiles,
-               scale * 1.4426950408889634f);
+               scale * 1.4426950408889634f, ext);
     SKN_LAUNCH_CHECK(ctx);
     return SKN_OK;
 }
@@ -252,12 +284,25 @@ int launch_prefill(skn_ctx* ctx, skn_kv* kv, int seq, const float* q_dev, int n_
 // (first_ctx >= 1; all of them must be cached).  head_dim 64 or 128.
 int skn_attn_prefill_launch(skn_ctx* ctx, skn_kv* kv, int seq, const float* q_dev, int n_queries, int first_ctx, float scale,
                             float* out_dev, int n_q_head) {
+    SKN_REQUIRE(ctx, !kv->shared, SKN_ERR_STATE, "attention: the cache shares its keys and values (skn_attn_shared reads it)");
     if (n_q_head <= 0) n_q_head = kv->n_head;
     SKN_REQUIRE(ctx, n_q_head % kv->n_head == 0, SKN_ERR_SHAPE,
                 "attention: %d query heads are not a multiple of the %d cached heads", n_q_head, kv->n_head);
-    if (kv->head_dim == 64) return launch_prefill<64>(ctx, kv, seq, q_dev, n_queries, first_ctx, scale, out_dev, n_q_head);
-    if (kv->head_dim == 128) return launch_prefill<128>(ctx, kv, seq, q_dev, n_queries, first_ctx, scale, out_dev, n_q_head);
+    if (kv->head_dim == 64) return launch_prefill<64, false>(ctx, kv, seq, q_dev, n_queries, first_ctx, scale, out_dev, n_q_head);
+    if (kv->head_dim == 128) return launch_prefill<128, false>(ctx, kv, seq, q_dev, n_queries, first_ctx, scale, out_dev, n_q_head);
     return skn_fail(ctx, SKN_ERR_SHAPE, "skn_attn_prefill: head_dim %d is not supported (64 or 128)", kv->head_dim);
+}
+
+int skn_shared_attn_prefill_launch(skn_ctx* ctx, skn_kv* kv, int seq, const float* q_prep, int n_queries, int first_ctx, int n_head, float scale,
+                                   void* out, int ldo, int out_type) {
+    SKN_REQUIRE(ctx, kv->shared && kv->elem_type == SKN_TYPE_F16 && n_head % kv->n_head == 0, SKN_ERR_STATE, "prompt attention: not a shared fp16 cache");
+    PrefillExt ext;
+    ext.dim = kv->dim;
+    ext.ldo = ldo;
+    ext.out_type = out_type;
+    if (kv->head_dim == 64) return launch_prefill<64, true>(ctx, kv, seq, q_prep, n_queries, first_ctx, scale, (float*)out, n_head, ext);
+    if (kv->head_dim == 128) return launch_prefill<128, true>(ctx, kv, seq, q_prep, n_queries, first_ctx, scale, (float*)out, n_head, ext);
+    return skn_fail(ctx, SKN_ERR_SHAPE, "prompt attention: head_dim %d is not supported (64 or 128)", kv->head_dim);
 }
 
 extern "C" int skn_attn_prefill(skn_ctx* ctx, skn_kv* kv, int seq, const float* q_dev, int n_queries, float scale,

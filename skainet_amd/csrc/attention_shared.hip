@@ -1,0 +1,424 @@
+// Attention whose values are its keys before their norm (one cached row per token and key head), with RMS norm of query
+// and key over their whole projections, a query temperature by position and a linear distance bias:
+//
+//   q' = q / rms(q) * q_norm * (1 + coef ln(floor((p + 1) / every) + 1)),   k' = k / rms(k) * k_norm,   v = k
+//   out_i = softmax_j <= i ( scale q'_i . k'_j - slope_h (i - j) ) v_j,      slope_h = 2^(-8 (h + 1) / n_head)
+//
+// The cache keeps the projected k (fp16 or fp32) and one factor 1 / rms(k) per token: the norm weights of the key go to the
+// query side (q' . k' = (q' k_norm) . k / rms(k)), so a row serves as key and as value and is read once for both -- and
+// once for all query heads of its group, whose queries a workgroup holds together.
+//
+// Token streams as in csrc/attention.hip: a row is spread over head_dim / 8 lanes, the lanes of a row own a private softmax
+// stream per query head, nothing is staged and no barrier is met while tokens stream.  A step's launch computes the two
+// norms of its own token in its prologue (every workgroup for itself, from L2) while its first rows are on their way.
+#include "dense.h"
+#include "kv.h"
+
+#include <algorithm>
+
+namespace {
+
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+typedef _Float16 half2_t __attribute__((ext_vector_type(2)));
+
+constexpr int kThreads = 512, kWaves = kThreads / 64;
+constexpr int kU = 4;           // rows per stream in flight
+constexpr int kMaxSplits = 16;  // what the merge in the output projection's staging is fed at most
+constexpr float kLog2e = 1.4426950408889634f;
+
+template <typename E>
+struct Row8;  // eight elements of a cached row
+template <>
+struct Row8<uint16_t> {
+    u32x4 a;
+    __device__ __forceinline__ void load(const uint16_t* p) { a = *reinterpret_cast<const u32x4*>(p); }
+    __device__ __forceinline__ void get(float (&f)[8]) const {
+#pragma unroll
+        for (int j = 0; j < 4; j++) {
+            const uint32_t w = a[j];  // (a bit cast applied directly to a vector element reads element 0)
+            const half2_t h = __builtin_bit_cast(half2_t, w);
+            f[2 * j] = (float)h.x;
+            f[2 * j + 1] = (float)h.y;
+        }
+    }
+};
+template <>
+struct Row8<float> {
+    float4 a, b;
+    __device__ __forceinline__ void load(const float* p) {
+        a = *reinterpret_cast<const float4*>(p);
+        b = *reinterpret_cast<const float4*>(p + 4);
+    }
+    __device__ __forceinline__ void get(float (&f)[8]) const {
+        f[0] = a.x, f[1] = a.y, f[2] = a.z, f[3] = a.w, f[4] = b.x, f[5] = b.y, f[6] = b.z, f[7] = b.w;
+    }
+};
+
+__device__ __forceinline__ float query_temperature(int pos, float coef, float every) {
+    return coef == 0.f ? 1.f : fmaf(coef, logf((float)floor((double)(pos + 1) / (double)every) + 1.0f), 1.0f);
+}
+
+struct AttnArgs {
+    const void* pool;
+    float* key_scale;
+    const int32_t* table;  // the sequence's row of the page table
+    int page_tokens, pages_per_seq, n_head, kv_heads, dim;
+    float scale_log2e;
+    int n_splits;
+    float* opart;
+    float* ml;
+    void* out;
+    int ldo, out_type;
+    // rows of a prompt: prepared queries, row z sees first_ctx + z tokens
+    const float* q_prep;
+    int first_ctx;
+    // one token: raw projections and their norms
+    const float* q;
+    const float* k;
+    const float* q_norm;
+    const float* k_norm;
+    const int32_t* state;
+    float eps, temp_coef, temp_every;
+};
+
+// sum of squares of x[0, n) over the workgroup; red: one float per wavefront (a barrier inside)
+__device__ __forceinline__ void block_sum_squares2(const float* x, int n, const float* y, int m, float* red, float& sx, float& sy) {
+    float a = 0.f, b = 0.f;
+    for (int i = threadIdx.x; i < n; i += blockDim.x) a = fmaf(x[i], x[i], a);
+    for (int i = threadIdx.x; i < m; i += blockDim.x) b = fmaf(y[i], y[i], b);
+    a = wave_sum(a);
+    b = wave_sum(b);
+    const int wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+    if ((threadIdx.x & 63) == 0) red[wave] = a, red[nw + wave] = b;
+    __syncthreads();
+    sx = sy = 0.f;
+    for (int i = 0; i < nw; i++) sx += red[i], sy += red[nw + i];
+}
+
+// grid (splits, kv heads x head groups, query rows)
+template <typename E, int D, int QG, bool STEP>
+__global__ __launch_bounds__(kThreads) void shared_attn_kernel(const AttnArgs p) {
+    constexpr int LPT = D / 8, G = 64 / LPT, NS = kWaves * G, U = kU;
+    __shared__ float so[kWaves][QG][D];
+    __shared__ float sm[kWaves][QG], sl[kWaves][QG];
+    __shared__ float red[2 * kWaves];
+    const int split = blockIdx.x, row = blockIdx.z;
+    const int per_kv = p.n_head / p.kv_heads, n_groups = (per_kv + QG - 1) / QG;
+    const int kvh = blockIdx.y / n_groups, h0 = kvh * per_kv + (blockIdx.y % n_groups) * QG, h_end = (kvh + 1) * per_kv;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int c = lane % LPT, g = lane / LPT, stream = wave * G + g;
+    const int n = STEP ? p.state[2] : p.first_ctx + row;
+    const int per = ((n + p.n_splits - 1) / p.n_splits + NS - 1) / NS * NS;
+    const int t_begin = split * per, t_end = min(n, t_begin + per);
+    const E* pool = (const E*)p.pool;
+    // the first 64 page ids ride in a register (lane i holds page i)
+    const int my_page = p.table[min(lane, p.pages_per_seq - 1)];
+
+    Row8<E> cur[U], nxt[U];
+    float cs_cur[U], cs_nxt[U];
+    auto fetch = [&](Row8<E>(&rows)[U], float(&cs)[U], int base) __attribute__((always_inline)) {
+#pragma unroll
+        for (int u = 0; u < U; u++) {
+            const int t = max(min(base + u * NS + stream, t_end - 1), 0);  // past the end: a valid row, masked below
+            const int pi = t / p.page_tokens, slot = t - pi * p.page_tokens;
+            int page = __shfl(my_page, pi & 63, 64);
+            if (pi >= 64) page = p.table[pi];
+            rows[u].load(pool + (((int64_t)page * p.kv_heads + kvh) * p.page_tokens + slot) * D + c * 8);
+            cs[u] = p.key_scale[(int64_t)page * p.page_tokens + slot];
+        }
+    };
+    if (t_begin < t_end) fetch(cur, cs_cur, t_begin);
+
+    float qf[QG][8], fq = p.scale_log2e, newest_scale = 0.f;
+    if constexpr (STEP) {
+        float sq, sk;
+        block_sum_squares2(p.q, p.n_head * p.dim, p.k, p.kv_heads * p.dim, red, sq, sk);
+        newest_scale = 1.0f / sqrtf(sk / (float)(p.kv_heads * p.dim) + p.eps);
+        fq *= query_temperature(n - 1, p.temp_coef, p.temp_every) / sqrtf(sq / (float)(p.n_head * p.dim) + p.eps);
+        if (split == 0 && blockIdx.y == 0 && tid == 0) {  // for the steps to come (this one uses its own)
+            const int pi = (n - 1) / p.page_tokens;
+            p.key_scale[(int64_t)p.table[pi] * p.page_tokens + (n - 1) - pi * p.page_tokens] = newest_scale;
+        }
+#pragma unroll
+        for (int i = 0; i < QG; i++) {
+            const int h = min(h0 + i, h_end - 1);
+#pragma unroll
+            for (int j = 0; j < 8; j++) {
+                const int d = c * 8 + j, at = min(d, p.dim - 1);
+                const float v = p.q[h * p.dim + at] * p.q_norm[h * p.dim + at] * p.k_norm[kvh * p.dim + at];
+                qf[i][j] = d < p.dim ? v : 0.f;
+            }
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < QG; i++) {
+            const float4* qp = reinterpret_cast<const float4*>(p.q_prep + ((int64_t)row * p.n_head + min(h0 + i, h_end - 1)) * D + c * 8);
+            const float4 a = qp[0], b = qp[1];
+            qf[i][0] = a.x, qf[i][1] = a.y, qf[i][2] = a.z, qf[i][3] = a.w, qf[i][4] = b.x, qf[i][5] = b.y, qf[i][6] = b.z, qf[i][7] = b.w;
+        }
+    }
+    float slope[QG], o[QG][8], m_run[QG], l_run[QG];
+#pragma unroll
+    for (int i = 0; i < QG; i++) {
+        slope[i] = exp2f(-8.0f * (float)(h0 + i + 1) / (float)p.n_head) * kLog2e;
+        m_run[i] = -INFINITY;
+        l_run[i] = 0.f;
+#pragma unroll
+        for (int j = 0; j < 8; j++) o[i][j] = 0.f;
+    }
+
+    auto absorb = [&](const Row8<E>(&rows)[U], const float(&cs)[U], int base) __attribute__((always_inline)) {
+        float sc[QG][U];
+#pragma unroll
+        for (int u = 0; u < U; u++) {
+            float kf[8];
+            rows[u].get(kf);
+            const int t = base + u * NS + stream;
+            const float f = (STEP && t == n - 1 ? newest_scale : cs[u]) * fq;
+            const float back = (float)(n - 1 - t);
+#pragma unroll
+            for (int i = 0; i < QG; i++) {
+                float d = 0.f;
+#pragma unroll
+                for (int j = 0; j < 8; j++) d = fmaf(kf[j], qf[i][j], d);
+                d = lane_group_sum<LPT>(d);
+                sc[i][u] = t < t_end ? fmaf(d, f, -slope[i] * back) : -INFINITY;
+            }
+        }
+        float pr[QG][U];
+#pragma unroll
+        for (int i = 0; i < QG; i++) {
+            float m_new = m_run[i];
+#pragma unroll
+            for (int u = 0; u < U; u++) m_new = fmaxf(m_new, sc[i][u]);
+            const float m_safe = m_new == -INFINITY ? 0.f : m_new;  // keeps exp2(-inf - -inf) out of the arithmetic
+            const float alpha = exp2f(m_run[i] - m_safe);
+            float sum = 0.f;
+#pragma unroll
+            for (int u = 0; u < U; u++) sum += pr[i][u] = exp2f(sc[i][u] - m_safe);
+            l_run[i] = fmaf(l_run[i], alpha, sum);
+            m_run[i] = m_new;
+#pragma unroll
+            for (int j = 0; j < 8; j++) o[i][j] *= alpha;
+        }
+#pragma unroll
+        for (int u = 0; u < U; u++) {
+            float vf[8];
+            rows[u].get(vf);
+#pragma unroll
+            for (int i = 0; i < QG; i++)
+#pragma unroll
+                for (int j = 0; j < 8; j++) o[i][j] = fmaf(pr[i][u], vf[j], o[i][j]);
+        }
+    };
+    for (int base = t_begin; base < t_end; base += 2 * NS * U) {
+        fetch(nxt, cs_nxt, base + NS * U);
+        absorb(cur, cs_cur, base);
+        fetch(cur, cs_cur, base + 2 * NS * U);
+        absorb(nxt, cs_nxt, base + NS * U);
+    }
+
+    // the G streams of the wavefront (lanes with the same c hold the same elements), then the wavefronts through LDS
+#pragma unroll
+    for (int i = 0; i < QG; i++) {
+        float mw = m_run[i];
+#pragma unroll
+        for (int off = LPT; off < 64; off <<= 1) mw = fmaxf(mw, __shfl_xor(mw, off, 64));
+        const float w = exp2f(m_run[i] - (mw == -INFINITY ? 0.f : mw));  // (an empty stream: exp2(-inf) = 0)
+        float lw = l_run[i] * w;
+#pragma unroll
+        for (int j = 0; j < 8; j++) o[i][j] *= w;
+#pragma unroll
+        for (int off = LPT; off < 64; off <<= 1) {
+            lw += __shfl_xor(lw, off, 64);
+#pragma unroll
+            for (int j = 0; j < 8; j++) o[i][j] += __shfl_xor(o[i][j], off, 64);
+        }
+        if (g == 0) {
+#pragma unroll
+            for (int j = 0; j < 8; j++) so[wave][i][c * 8 + j] = o[i][j];
+            if (c == 0) sm[wave][i] = mw, sl[wave][i] = lw;
+        }
+    }
+    __syncthreads();
+    for (int e = tid; e < QG * D; e += kThreads) {
+        const int i = e / D, d = e - i * D, h = h0 + i;
+        if (h >= h_end) continue;
+        float m = -INFINITY, acc = 0.f, l = 0.f;
+#pragma unroll
+        for (int w = 0; w < kWaves; w++) m = fmaxf(m, sm[w][i]);
+        const float m_safe = m == -INFINITY ? 0.f : m;
+#pragma unroll
+        for (int w = 0; w < kWaves; w++) {
+            const float f = exp2f(sm[w][i] - m_safe);
+            acc = fmaf(f, so[w][i][d], acc);
+            l = fmaf(f, sl[w][i], l);
+        }
+        if (p.n_splits > 1) {
+            p.opart[((int64_t)split * p.n_head + h) * D + d] = acc;
+            if (d == 0) p.ml[2 * (split * p.n_head + h)] = m, p.ml[2 * (split * p.n_head + h) + 1] = l;
+        } else if (d < p.dim) {
+            const float v = acc / l;
+            const int64_t at = (int64_t)row * p.ldo + h * p.dim + d;
+            if (p.out_type == SKN_TYPE_F32) ((float*)p.out)[at] = v;
+            else ((uint16_t*)p.out)[at] = skn_bf16_bits(v);
+        }
+    }
+}
+
+// one workgroup per row: norms, temperature, the query in its padded layout with the key's norm weights, the key to the cache
+template <typename E>
+__global__ __launch_bounds__(256) void shared_prep_kernel(const float* __restrict__ q, int ldq, const float* __restrict__ k, int ldk,
+                                                          const float* __restrict__ q_norm, const float* __restrict__ k_norm, E* __restrict__ pool,
+                                                          float* __restrict__ key_scale, const int32_t* __restrict__ table, int page_tokens,
+                                                          int n_head, int kv_heads, int dim, int dim_pad, int pos0, float eps, float temp_coef,
+                                                          float temp_every, float* __restrict__ q_prep) {
+    __shared__ float red[8];
+    const int row = blockIdx.x, pos = pos0 + row;
+    const float* qr = q + (int64_t)row * ldq;
+    const float* kr = k + (int64_t)row * ldk;
+    float sq, sk;
+    block_sum_squares2(qr, n_head * dim, kr, kv_heads * dim, red, sq, sk);
+    const float rk = 1.0f / sqrtf(sk / (float)(kv_heads * dim) + eps);
+    const float rq = query_temperature(pos, temp_coef, temp_every) / sqrtf(sq / (float)(n_head * dim) + eps);
+    const int page = table[pos / page_tokens], slot = pos % page_tokens, per_kv = n_head / kv_heads;
+    if (threadIdx.x == 0) key_scale[(int64_t)page * page_tokens + slot] = rk;
+    for (int e = threadIdx.x; e < n_head * dim_pad; e += 256) {
+        const int h = e / dim_pad, d = e - h * dim_pad;
+        q_prep[(int64_t)row * n_head * dim_pad + e] =
+            d < dim ? qr[h * dim + d] * rq * q_norm[h * dim + d] * k_norm[h / per_kv * dim + d] : 0.f;
+    }
+    for (int e = threadIdx.x; e < kv_heads * dim; e += 256) {
+        const int h = e / dim, d = e - h * dim;
+        const int64_t at = (((int64_t)page * kv_heads + h) * page_tokens + slot) * dim_pad + d;
+        if constexpr (sizeof(E) == 4) pool[at] = kr[e];
+        else pool[at] = __half_as_ushort(__float2half_rn(kr[e]));
+    }
+}
+
+template <typename E, int D, bool STEP>
+int launch_qg(skn_ctx* ctx, const AttnArgs& a, int rows) {
+    const int per_kv = a.n_head / a.kv_heads;
+    auto grid = [&](int qg) { return dim3(a.n_splits, a.kv_heads * ((per_kv + qg - 1) / qg), rows); };
+    if (per_kv == 1) skn_launch(ctx, shared_attn_kernel<E, D, 1, STEP>, grid(1), dim3(kThreads), 0, a);
+    else if (per_kv == 2) skn_launch(ctx, shared_attn_kernel<E, D, 2, STEP>, grid(2), dim3(kThreads), 0, a);
+    else skn_launch(ctx, shared_attn_kernel<E, D, 4, STEP>, grid(4), dim3(kThreads), 0, a);
+    SKN_LAUNCH_CHECK(ctx);
+    return SKN_OK;
+}
+
+template <bool STEP>
+int launch_attn(skn_ctx* ctx, const skn_kv* kv, const AttnArgs& a, int rows) {
+    const bool f32 = kv->elem_type == SKN_TYPE_F32;
+    switch (kv->head_dim) {
+        case 64: return f32 ? launch_qg<float, 64, STEP>(ctx, a, rows) : launch_qg<uint16_t, 64, STEP>(ctx, a, rows);
+        case 128: return f32 ? launch_qg<float, 128, STEP>(ctx, a, rows) : launch_qg<uint16_t, 128, STEP>(ctx, a, rows);
+        default: return f32 ? launch_qg<float, 256, STEP>(ctx, a, rows) : launch_qg<uint16_t, 256, STEP>(ctx, a, rows);
+    }
+}
+
+AttnArgs base_args(const skn_kv* kv, int seq, const skn_shared_attn& p) {
+    AttnArgs a = {};
+    a.pool = kv->k_pool;
+    a.key_scale = kv->key_scale;
+    a.table = kv->page_table_dev + (size_t)seq * kv->pages_per_seq;
+    a.page_tokens = kv->page_tokens;
+    a.pages_per_seq = kv->pages_per_seq;
+    a.n_head = p.n_head;
+    a.kv_heads = kv->n_head;
+    a.dim = kv->dim;
+    a.scale_log2e = p.scale * kLog2e;
+    a.n_splits = 1;
+    a.q_norm = p.q_norm;
+    a.k_norm = p.k_norm;
+    a.eps = p.eps;
+    a.temp_coef = p.temp_coef;
+    a.temp_every = p.temp_every;
+    return a;
+}
+
+int check(skn_ctx* ctx, const skn_kv* kv, const skn_shared_attn& p) {
+    SKN_REQUIRE(ctx, kv->shared, SKN_ERR_STATE, "shared attention: the cache keeps keys and values apart");
+    SKN_REQUIRE(ctx, p.n_head > 0 && p.n_head % kv->n_head == 0, SKN_ERR_SHAPE, "shared attention: %d query heads over %d cached heads", p.n_head, kv->n_head);
+    SKN_REQUIRE(ctx, p.q_norm && p.k_norm && (p.temp_coef == 0.f || p.temp_every > 0.f), SKN_ERR_ARG, "shared attention: bad parameters");
+    return SKN_OK;
+}
+
+}  // namespace
+
+int skn_shared_prep_rows(skn_ctx* ctx, skn_kv* kv, int seq, const skn_shared_attn& p, const float* q, int ldq, const float* k, int ldk, int n,
+                         int pos0, float* q_prep) {
+    SKN_TRY(check(ctx, kv, p));
+    const int32_t* table = kv->page_table_dev + (size_t)seq * kv->pages_per_seq;
+    if (kv->elem_type == SKN_TYPE_F32)
+        skn_launch(ctx, shared_prep_kernel<float>, dim3(n), dim3(256), 0, q, ldq, k, ldk, p.q_norm, p.k_norm, (float*)kv->k_pool, kv->key_scale, table,
+                   kv->page_tokens, p.n_head, kv->n_head, kv->dim, kv->head_dim, pos0, p.eps, p.temp_coef, p.temp_every, q_prep);
+    else
+        skn_launch(ctx, shared_prep_kernel<uint16_t>, dim3(n), dim3(256), 0, q, ldq, k, ldk, p.q_norm, p.k_norm, kv->k_pool, kv->key_scale, table,
+                   kv->page_tokens, p.n_head, kv->n_head, kv->dim, kv->head_dim, pos0, p.eps, p.temp_coef, p.temp_every, q_prep);
+    SKN_LAUNCH_CHECK(ctx);
+    return SKN_OK;
+}
+
+int skn_shared_attn_rows(skn_ctx* ctx, skn_kv* kv, int seq, const skn_shared_attn& p, const float* q_prep, int n, int pos0, void* out, int ldo,
+                         int out_type) {
+    SKN_TRY(check(ctx, kv, p));
+    if (kv->elem_type == SKN_TYPE_F16 && kv->head_dim <= 128)
+        return skn_shared_attn_prefill_launch(ctx, kv, seq, q_prep, n, pos0 + 1, p.n_head, p.scale, out, ldo, out_type);
+    AttnArgs a = base_args(kv, seq, p);
+    a.out = out;
+    a.ldo = ldo;
+    a.out_type = out_type;
+    for (int z = 0; z < n; z += 32768) {  // (grid limit)
+        a.q_prep = q_prep + (int64_t)z * p.n_head * kv->head_dim;
+        a.first_ctx = pos0 + z + 1;
+        a.out = (uint8_t*)out + (int64_t)z * ldo * (out_type == SKN_TYPE_F32 ? 4 : 2);
+        SKN_TRY(launch_attn<false>(ctx, kv, a, std::min(n - z, 32768)));
+    }
+    return SKN_OK;
+}
+
+int skn_shared_attn_step(skn_ctx* ctx, skn_kv* kv, int seq, const skn_shared_attn& p, const float* q, const float* k, const int32_t* state_dev,
+                         int n_splits, float* opart, float* ml, float* out) {
+    SKN_TRY(check(ctx, kv, p));
+    SKN_REQUIRE(ctx, n_splits >= 1 && n_splits <= kMaxSplits && (n_splits == 1 ? out != nullptr : opart && ml), SKN_ERR_ARG,
+                "shared attention: %d splits without their buffers", n_splits);
+    AttnArgs a = base_args(kv, seq, p);
+    a.q = q;
+    a.k = k;
+    a.state = state_dev;
+    a.n_splits = n_splits;
+    a.opart = opart;
+    a.ml = ml;
+    a.out = out;
+    a.out_type = SKN_TYPE_F32;
+    return launch_attn<true>(ctx, kv, a, 1);
+}
+
+// Splits for contexts up to max_ctx: a power of two, so that a workgroup has at least two rounds of requests and the
+// workgroups do not outnumber the compute units (the merge reads every split in every workgroup that follows).
+int skn_shared_attn_splits(skn_ctx* ctx, const skn_kv* kv, int n_head, int max_ctx) {
+    const int per_kv = n_head / kv->n_head, qg = per_kv >= 4 ? 4 : per_kv >= 2 ? 2 : 1;
+    const int wgs = kv->n_head * ((per_kv + qg - 1) / qg), round = kWaves * 512 / kv->head_dim * kU;
+    int n = 1;
+    while (n < kMaxSplits && n * round < max_ctx && 2 * n * wgs <= ctx->compute_units) n *= 2;
+    return n;
+}
+
+extern "C" int skn_attn_shared(skn_ctx* ctx, skn_kv* kv, int seq, const skn_shared_attn* p, const float* q_dev, const float* k_dev, int n,
+                               float* out_dev) {
+    SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_attn_shared: ctx is null");
+    SKN_REQUIRE(ctx, kv && p && q_dev && k_dev && out_dev, SKN_ERR_ARG, "skn_attn_shared: null pointer");
+    SKN_REQUIRE(ctx, seq >= 0 && seq < kv->n_seq && n > 0, SKN_ERR_RANGE, "skn_attn_shared: %d tokens of sequence %d of %d", n, seq, kv->n_seq);
+    SKN_TRY(check(ctx, kv, *p));
+    const int pos0 = kv->len[seq];
+    SKN_TRY(skn_kv_reserve(ctx, kv, seq, pos0 + n));
+    float* q_prep = nullptr;
+    SKN_HIP(ctx, hipMalloc((void**)&q_prep, (size_t)n * p->n_head * kv->head_dim * sizeof(float)));
+    int rc = skn_shared_prep_rows(ctx, kv, seq, *p, q_dev, p->n_head * kv->dim, k_dev, kv->n_head * kv->dim, n, pos0, q_prep);
+    if (rc == SKN_OK) rc = skn_shared_attn_rows(ctx, kv, seq, *p, q_prep, n, pos0, out_dev, p->n_head * kv->dim, SKN_TYPE_F32);
+    if (rc == SKN_OK) rc = skn_kv_advance_len(ctx, kv, seq, n);
+    (void)hipStreamSynchronize(ctx->stream);
+    (void)hipFree(q_prep);
+    return rc;
+}

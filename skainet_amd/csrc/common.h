@@ -29,7 +29,7 @@ struct skn_ctx {
     std::vector<hipEvent_t> prof_events;
     // tuning options (skn_set_option); 0 = library default
     int opt_q4k_split = 0;  // Q4_K matvec with k split across workgroups (measured alternative): 1 ticket merge, 2 atomic adds
-    int opt_q4k_waves = 0, opt_q4k_rows = 0, opt_attn_splits = 0, opt_llama_graph = 1, opt_llama_fused = 1, opt_gemm_tile = 0, opt_matvec_stage = 1, opt_llama_expand = 0, opt_test_rope_table = 0, opt_llama_attn_wide = 1, opt_gemm_q6k_fused = 1;
+    int opt_q4k_waves = 0, opt_q4k_rows = 0, opt_attn_splits = 0, opt_llama_graph = 1, opt_llama_fused = 1, opt_gemm_tile = 0, opt_matvec_stage = 1, opt_llama_expand = 0, opt_test_rope_table = 0, opt_llama_attn_wide = 1, opt_gemm_q6k_fused = 1, opt_dense_tile = 0;
     int opt_generation = 0;          // bumped by every skn_set_option / skn_set_stream: captured work is stamped with it
     bool profiler_attached = false;  // a rocprofiler tool library is loaded into this process: graphs are not replayed
     long long stat_launches = 0, stat_captures = 0;  // kernel launches issued (or recorded) / decode-step graphs captured
@@ -51,10 +51,12 @@ struct skn_ctx {
     size_t gemm_ws_bytes = 0;
 };
 
-// One-time kernel attribute setup (large dynamic LDS), called by skn_init.
-int skn_matvec_init(skn_ctx* ctx);
-int skn_gemm_init(skn_ctx* ctx);
-int skn_attn_init(skn_ctx* ctx);
+// One-time setup of a kernel family (large dynamic LDS, static scratch): a source file that needs some registers its
+// function with an object of this type at namespace scope, and skn_init calls every registered one.  (The library can be
+// linked from any set of families.)
+struct skn_family {
+    explicit skn_family(int (*init)(skn_ctx* ctx));
+};
 
 // Fused Q4_K matvec used by the decoder: up to three [rows_i, k] matrices stacked along the output axis,
 // optional RMSNorm of x (norm_w != nullptr) and a store / add-into / SwiGLU epilogue.
@@ -105,6 +107,12 @@ int skn_fail(skn_ctx* ctx, int code, const char* fmt, ...);
         if (e_ != hipSuccess)                                                                          \
             return skn_fail((ctx), SKN_ERR_HIP, "%s failed: %s (%s:%d)", #expr, hipGetErrorString(e_), \
                             __FILE__, __LINE__);                                                       \
+    } while (0)
+
+#define SKN_TRY(expr)              \
+    do {                           \
+        int rc_ = (expr);          \
+        if (rc_ != SKN_OK) return rc_; \
     } while (0)
 
 // Call after a kernel launch.
@@ -246,6 +254,18 @@ __device__ __forceinline__ float row16_sum(float v) {
     v += __int_as_float(i);
     i = __builtin_amdgcn_mov_dpp(__float_as_int(v), 0x140, 0xF, 0xF, true);
     v += __int_as_float(i);
+    return v;
+}
+
+// Sum over each aligned group of N = 4, 8, 16 or 32 lanes; every lane of the group returns its group's total.
+template <int N>
+__device__ __forceinline__ float lane_group_sum(float v) {
+    static_assert(N == 4 || N == 8 || N == 16 || N == 32, "group of 4, 8, 16 or 32 lanes");
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, true));   // lane ^ 1
+    v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x4E, 0xF, 0xF, true));   // lane ^ 2
+    if constexpr (N >= 8) v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x141, 0xF, 0xF, true));  // 7 - lane
+    if constexpr (N >= 16) v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x140, 0xF, 0xF, true));
+    if constexpr (N >= 32) v += __shfl_xor(v, 16, 64);
     return v;
 }
 

@@ -1,12 +1,10 @@
 // Llama-style decoder over the quantized kernels: batched prompt processing (GEMM) and greedy decode (matvec)
 // for one sequence.  Per layer:  x += Wo . attn(rope(Wq xn), cache(rope(Wk xn), Wv xn)),  xn = rmsnorm(x);
 // x += Wdown . (silu(Wgate xn) * (Wup xn)).  Logits = Whead . rmsnorm(x).
-//
-// A decode step reads every scalar that changes from step to step (token id, position, context length, step
-// index) from device memory, so that one captured HIP graph of the ~480 kernel launches of a step can be
-// replayed for every token.  The graph holds kernels only (no memset / memcpy nodes).
+// The decode loop around a step (device scalars, greedy choice, captured graph) is csrc/stepper.h.
 #include "kv.h"
 #include "gemm_q6k.h"
+#include "stepper.h"
 
 #include <algorithm>
 #include <cmath>
@@ -20,10 +18,8 @@ struct skn_llama {
     float *x = nullptr, *xn = nullptr, *q = nullptr, *k = nullptr, *v = nullptr, *att = nullptr, *proj = nullptr;
     float *gate = nullptr, *up = nullptr, *mid = nullptr, *logits = nullptr, *attn_partial = nullptr;
     int *attn_counters = nullptr, *pcounters = nullptr;  // split counters of the attention launches (zero between launches)
-    int32_t* state = nullptr;       // [0] token, [1] position, [2] context length, [3] step index
-    int32_t* tokens_out = nullptr;  // device array of produced tokens
+    skn_stepper step;
     double* inv_freq = nullptr;     // rope_base^(-2i / head_dim), i < head_dim / 2, formed in double on the host
-    int tokens_cap = 0;
     int pos = 0;                    // host mirror of the position
     // prompt buffers (grown to the longest prompt seen)
     int prompt_cap = 0;
@@ -31,11 +27,6 @@ struct skn_llama {
     float *pgate = nullptr, *pup = nullptr, *pmid = nullptr, *ppartial = nullptr;
     uint16_t *pb16 = nullptr, *pk16 = nullptr, *pv16 = nullptr;
     int32_t *ptok = nullptr, *pnctx = nullptr;
-    // captured decode step
-    hipGraph_t graph = nullptr;
-    hipGraphExec_t graph_exec = nullptr;
-    int graph_splits = 0;
-    int graph_generation = -1;  // ctx->opt_generation at capture: every option decode_step reads, and the stream
     // fp16-pair copies of the matrices that are not Q4_K, for the prompt GEMMs (made on first use when the option
     // llama.expand_weights is set): seven per layer in the order q, k, v, o, gate, up, down
     std::vector<void*> expanded;
@@ -200,79 +191,6 @@ __global__ void f32_to_bf16_rows_kernel(const float* __restrict__ x, uint16_t* _
     }
 }
 
-// state = {token, position, context length, step}
-__global__ void set_state_kernel(int32_t* state, int token, int pos) {
-    if (threadIdx.x == 0) {
-        state[0] = token;
-        state[1] = pos;
-        state[2] = pos + 1;
-        state[3] = 0;
-    }
-}
-
-// single workgroup: argmax of the logits (first maximum) becomes the next token; the step's scalars advance
-__global__ __launch_bounds__(1024) void finish_step_kernel(const float* __restrict__ x, int n, int32_t* state,
-                                                           int32_t* __restrict__ tokens_out, int advance) {
-    __shared__ float bv[16];
-    __shared__ int bi[16];
-    float best = -INFINITY;
-    int besti = 0x7FFFFFFF;
-    auto take = [&](float v, int i) {
-        if (v > best || (v == best && i < besti)) {
-            best = v;
-            besti = i;
-        }
-    };
-    // eight float4 per thread and round, all loaded before the first compare
-    const int n4 = n >> 2;
-    for (int base = 0; base < n4; base += 8 * 1024) {
-        float4 v[8];
-#pragma unroll
-        for (int j = 0; j < 8; j++) v[j] = reinterpret_cast<const float4*>(x)[min(base + j * 1024 + (int)threadIdx.x, n4 - 1)];
-#pragma unroll
-        for (int j = 0; j < 8; j++) {
-            const int i4 = base + j * 1024 + (int)threadIdx.x;
-            if (i4 < n4) {
-                take(v[j].x, 4 * i4);
-                take(v[j].y, 4 * i4 + 1);
-                take(v[j].z, 4 * i4 + 2);
-                take(v[j].w, 4 * i4 + 3);
-            }
-        }
-    }
-    for (int i = 4 * n4 + threadIdx.x; i < n; i += 1024) take(x[i], i);
-    for (int off = 32; off >= 1; off >>= 1) {
-        const float ov = __shfl_xor(best, off, 64);
-        const int oi = __shfl_xor(besti, off, 64);
-        if (ov > best || (ov == best && oi < besti)) {
-            best = ov;
-            besti = oi;
-        }
-    }
-    if ((threadIdx.x & 63) == 0) {
-        bv[threadIdx.x >> 6] = best;
-        bi[threadIdx.x >> 6] = besti;
-    }
-    __syncthreads();
-    if (threadIdx.x == 0) {
-        for (int w = 1; w < 16; w++)
-            if (bv[w] > best || (bv[w] == best && bi[w] < besti)) {
-                best = bv[w];
-                besti = bi[w];
-            }
-        const int tok = besti == 0x7FFFFFFF ? 0 : besti;
-        if (advance) {
-            tokens_out[state[3]] = tok;
-            state[0] = tok;
-            state[1] += 1;
-            state[2] += 1;
-            state[3] += 1;
-        } else {
-            tokens_out[0] = tok;
-        }
-    }
-}
-
 __global__ void iota_kernel(int32_t* out, int n, int start) {
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (i < n) out[i] = start + i;
@@ -291,19 +209,13 @@ int dev_alloc(skn_ctx* ctx, skn_llama* m, T** p, size_t count) {
 
 unsigned nblk(int64_t n) { return (unsigned)((n + 255) / 256); }
 
-#define SKN_TRY(expr)              \
-    do {                           \
-        int rc_ = (expr);          \
-        if (rc_ != SKN_OK) return rc_; \
-    } while (0)
-
 // the launches of one decode step (eagerly or under stream capture)
 int decode_step(skn_ctx* ctx, skn_llama* m, int n_splits) {
     const skn_llama_config& c = m->cfg;
     const int H = c.hidden, F = c.ffn, NH = c.n_head, D = c.head_dim, KVH = c.n_kv_head, KVD = KVH * D;
     const float scale = 1.0f / sqrtf((float)D);
     skn_launch(ctx, embed_rows_kernel, dim3(1), dim3(1024), 0, (const uint8_t*)m->w.tok_embd, m->w.type_embd, H,
-               (const int32_t*)m->state, m->x);
+               (const int32_t*)m->step.state, m->x);
     SKN_LAUNCH_CHECK(ctx);
     for (int l = 0; l < c.n_layer; l++) {
         const skn_llama_layer& L = m->layers[l];
@@ -320,7 +232,7 @@ int decode_step(skn_ctx* ctx, skn_llama* m, int n_splits) {
         const bool f_down = ctx->opt_llama_fused && F <= 16384 && F % 256 == 0 && skn_matvec_fusable(L.type_down);
         if (f_qkv) {
             skn_rope_epilogue rope;
-            rope.pos_dev = m->state + 1;
+            rope.pos_dev = m->step.state + 1;
             rope.page_table = kv->page_table_dev;
             rope.k_pool = kv->k_pool;
             rope.v_pool = kv->v_pool;
@@ -347,7 +259,7 @@ int decode_step(skn_ctx* ctx, skn_llama* m, int n_splits) {
             SKN_TRY(skn_matvec_q(ctx, L.type_k, L.wk, KVD, H, m->xn, m->k));
             SKN_TRY(skn_matvec_q(ctx, L.type_v, L.wv, KVD, H, m->xn, m->v));
             skn_launch(ctx, rope_store_kernel, dim3(1, NH), dim3(D / 2), 0, m->q, (const float*)m->k, (const float*)m->v,
-                       kv->k_pool, kv->v_pool, (const int32_t*)kv->page_table_dev, (const int32_t*)(m->state + 1), NH, KVH, D,
+                       kv->k_pool, kv->v_pool, (const int32_t*)kv->page_table_dev, (const int32_t*)(m->step.state + 1), NH, KVH, D,
                        kv->page_tokens, log2((double)c.rope_base));
             SKN_LAUNCH_CHECK(ctx);
         }
@@ -361,7 +273,7 @@ int decode_step(skn_ctx* ctx, skn_llama* m, int n_splits) {
             if (ctx->opt_llama_attn_wide > 1) wide = std::min(wide, ctx->opt_llama_attn_wide);  // (tuning: 2, 4 or 8 caps the count)
             float* opart = m->attn_partial;
             float* ml = m->attn_partial + (size_t)wide * NH * D;
-            SKN_TRY(skn_attn_launch_unmerged(ctx, kv, m->q, m->state + 2, 1, 0, wide, opart, ml, scale, m->att, NH));
+            SKN_TRY(skn_attn_launch_unmerged(ctx, kv, m->q, m->step.state + 2, 1, 0, wide, opart, ml, scale, m->att, NH));
             skn_q4k_segments wo = {{(const uint8_t*)L.wo, nullptr, nullptr}, {H, 0, 0}};
             skn_rope_epilogue mg;
             mg.merge_ml = ml;
@@ -370,11 +282,11 @@ int decode_step(skn_ctx* ctx, skn_llama* m, int n_splits) {
             mg.merge_head_f4 = D / 4;
             SKN_TRY(skn_matvec_q4k_fused(ctx, wo, H, H, opart, nullptr, 0.f, m->x, SKN_EPI_ADD, &mg, L.type_o));
         } else if (f_o) {
-            SKN_TRY(skn_attn_launch_ex(ctx, kv, m->q, m->state + 2, 1, 0, n_splits, m->attn_partial, m->attn_counters, scale, m->att, NH));
+            SKN_TRY(skn_attn_launch_ex(ctx, kv, m->q, m->step.state + 2, 1, 0, n_splits, m->attn_partial, m->attn_counters, scale, m->att, NH));
             skn_q4k_segments wo = {{(const uint8_t*)L.wo, nullptr, nullptr}, {H, 0, 0}};
             SKN_TRY(skn_matvec_q4k_fused(ctx, wo, H, H, m->att, nullptr, 0.f, m->x, SKN_EPI_ADD, nullptr, L.type_o));
         } else {
-            SKN_TRY(skn_attn_launch_ex(ctx, kv, m->q, m->state + 2, 1, 0, n_splits, m->attn_partial, m->attn_counters, scale, m->att, NH));
+            SKN_TRY(skn_attn_launch_ex(ctx, kv, m->q, m->step.state + 2, 1, 0, n_splits, m->attn_partial, m->attn_counters, scale, m->att, NH));
             SKN_TRY(skn_matvec_q(ctx, L.type_o, L.wo, H, H, m->att, m->proj));
             skn_launch(ctx, add_rows_kernel, dim3(nblk(H)), dim3(256), 0, m->x, (const float*)m->proj, (int64_t)H);
             SKN_LAUNCH_CHECK(ctx);
@@ -405,19 +317,7 @@ int decode_step(skn_ctx* ctx, skn_llama* m, int n_splits) {
     skn_launch(ctx, rmsnorm_rows_kernel, dim3(1), dim3(256), 0, (const float*)m->x, m->w.out_norm, m->xn, H, c.rms_eps);
     SKN_LAUNCH_CHECK(ctx);
     SKN_TRY(skn_matvec_q(ctx, m->w.type_head, m->w.out_head, c.vocab, H, m->xn, m->logits));
-    skn_launch(ctx, finish_step_kernel, dim3(1), dim3(1024), 0, (const float*)m->logits, c.vocab, m->state,
-               m->tokens_out, 1);
-    SKN_LAUNCH_CHECK(ctx);
-    return SKN_OK;
-}
-
-void drop_graph(skn_llama* m) {
-    if (m->graph_exec) (void)hipGraphExecDestroy(m->graph_exec);
-    if (m->graph) (void)hipGraphDestroy(m->graph);
-    m->graph_exec = nullptr;
-    m->graph = nullptr;
-    m->graph_splits = 0;
-    m->graph_generation = -1;
+    return skn_stepper_pick(ctx, &m->step, m->logits, c.vocab, 1);
 }
 
 // frees a buffer of the model now (the stream must be idle) and forgets it
@@ -540,7 +440,6 @@ int skn_llama_create(skn_ctx* ctx, const skn_llama_config* cfg, const skn_llama_
         (void)hipGetLastError();
         rc = skn_fail(ctx, SKN_ERR_HIP, "skn_llama_create: clearing the attention counters failed");
     }
-    A(&m->state, (size_t)4);
     A(&m->inv_freq, (size_t)cfg->head_dim / 2);
     if (rc == SKN_OK) {
         std::vector<double> f(cfg->head_dim / 2);
@@ -550,8 +449,7 @@ int skn_llama_create(skn_ctx* ctx, const skn_llama_config* cfg, const skn_llama_
             rc = skn_fail(ctx, SKN_ERR_HIP, "skn_llama_create: uploading the rotary frequencies failed");
         }
     }
-    m->tokens_cap = cfg->max_tokens;
-    A(&m->tokens_out, (size_t)m->tokens_cap);
+    if (rc == SKN_OK) rc = skn_stepper_create(ctx, &m->step, cfg->max_tokens);
     if (rc != SKN_OK) {
         skn_llama_free(ctx, m);
         return rc;
@@ -564,7 +462,7 @@ int skn_llama_free(skn_ctx* ctx, skn_llama* m) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_llama_free: ctx is null");
     if (!m) return SKN_OK;
     (void)hipStreamSynchronize(ctx->stream);
-    drop_graph(m);
+    skn_stepper_free(&m->step);
     for (skn_kv* kv : m->kv) skn_kv_free(ctx, kv);
     for (void* p : m->owned) (void)hipFree(p);
     ctx->stat_expanded_bytes -= m->expanded_bytes;
@@ -654,8 +552,7 @@ int skn_llama_prefill(skn_ctx* ctx, skn_llama* m, const int32_t* tokens_host, in
     SKN_TRY(ensure_prompt_buffers(ctx, m, T));
     SKN_HIP(ctx, hipMemcpyAsync(m->ptok, tokens_host, (size_t)T * sizeof(int32_t), hipMemcpyHostToDevice, ctx->stream));
     SKN_HIP(ctx, hipStreamSynchronize(ctx->stream));
-    skn_launch(ctx, set_state_kernel, dim3(1), dim3(64), 0, m->state, 0, pos0);
-    SKN_LAUNCH_CHECK(ctx);
+    SKN_TRY(skn_stepper_set(ctx, &m->step, 0, pos0));
     skn_launch(ctx, iota_kernel, dim3(nblk(T)), dim3(256), 0, m->pnctx, T, pos0 + 1);
     SKN_LAUNCH_CHECK(ctx);
     skn_launch(ctx, embed_rows_kernel, dim3(T), dim3(256), 0, (const uint8_t*)m->w.tok_embd, m->w.type_embd, H,
@@ -706,7 +603,7 @@ int skn_llama_prefill(skn_ctx* ctx, skn_llama* m, const int32_t* tokens_host, in
             SKN_TRY(project_rows(ctx, m, types, blocks, rows, outs, 3, H, m->px, L.attn_norm, T, 0));
         }
         skn_launch(ctx, rope_store_kernel, dim3(T, NH), dim3(D / 2), 0, m->pq, (const float*)m->pk, (const float*)m->pv,
-                   kv->k_pool, kv->v_pool, (const int32_t*)kv->page_table_dev, (const int32_t*)(m->state + 1), NH, KVH, D,
+                   kv->k_pool, kv->v_pool, (const int32_t*)kv->page_table_dev, (const int32_t*)(m->step.state + 1), NH, KVH, D,
                    kv->page_tokens, log2((double)c.rope_base));
         SKN_LAUNCH_CHECK(ctx);
         // query row t attends to the first pos0 + t + 1 tokens of the (single) sequence
@@ -780,12 +677,10 @@ int skn_llama_prefill(skn_ctx* ctx, skn_llama* m, const int32_t* tokens_host, in
                m->w.out_norm, m->xn, H, c.rms_eps);
     SKN_LAUNCH_CHECK(ctx);
     SKN_TRY(skn_matvec_q(ctx, m->w.type_head, m->w.out_head, c.vocab, H, m->xn, m->logits));
-    skn_launch(ctx, finish_step_kernel, dim3(1), dim3(1024), 0, (const float*)m->logits, c.vocab, m->state,
-               m->tokens_out, 0);
-    SKN_LAUNCH_CHECK(ctx);
+    SKN_TRY(skn_stepper_pick(ctx, &m->step, m->logits, c.vocab, 0));
     m->pos = pos0 + T;
     int32_t next = 0;
-    SKN_HIP(ctx, hipMemcpyAsync(&next, m->tokens_out, sizeof(int32_t), hipMemcpyDeviceToHost, ctx->stream));
+    SKN_HIP(ctx, hipMemcpyAsync(&next, m->step.tokens_out, sizeof(int32_t), hipMemcpyDeviceToHost, ctx->stream));
     SKN_HIP(ctx, hipStreamSynchronize(ctx->stream));
     if (next_token_host) *next_token_host = next;
     return SKN_OK;
@@ -802,11 +697,10 @@ int skn_llama_decode(skn_ctx* ctx, skn_llama* m, int32_t first_token, int n_step
                 "skn_llama_decode: token %d of a vocabulary of %d", first_token, c.vocab);
     SKN_REQUIRE(ctx, m->pos + n_steps <= c.max_tokens, SKN_ERR_POOL, "sequence is full (%d tokens, capacity %d)",
                 m->pos + n_steps, c.max_tokens);
-    SKN_REQUIRE(ctx, !ctx->prof_on, SKN_ERR_STATE, "skn_llama_decode: not available while per-launch timing is on");
+    SKN_REQUIRE(ctx, !ctx->prof_on || ctx->opt_llama_graph == 0, SKN_ERR_STATE,
+                "skn_llama_decode: not available while per-launch timing is on (except with llama.graph = 0)");
     // every page the run will touch is mapped now; the step itself never talks to the host
     for (skn_kv* kv : m->kv) SKN_TRY(skn_kv_reserve(ctx, kv, 0, m->pos + n_steps));
-    skn_launch(ctx, set_state_kernel, dim3(1), dim3(64), 0, m->state, (int)first_token, m->pos);
-    SKN_LAUNCH_CHECK(ctx);
     // A split count for the longest context of this run, rounded up to a power of two of 128-token units (the kernel
     // derives its ranges from the actual length, so one captured step serves every position up to there): the step is
     // captured again only when a sequence grows past 128, 256, 512, ... tokens, and a short context is not cut into
@@ -814,33 +708,8 @@ int skn_llama_decode(skn_ctx* ctx, skn_llama* m, int32_t first_token, int n_step
     int n_splits = 1;
     while (n_splits * 128 < m->pos + n_steps) n_splits *= 2;
     n_splits = std::min(n_splits, skn_attn_splits(ctx, c.n_head, c.max_tokens));
-    if (ctx->opt_llama_graph == 0) {
-        for (int i = 0; i < n_steps; i++) SKN_TRY(decode_step(ctx, m, n_splits));
-    } else {
-        // a captured step has the kernel set of the options (and the stream) it was captured with baked in
-        if (m->graph_exec && (m->graph_splits != n_splits || m->graph_generation != ctx->opt_generation)) drop_graph(m);
-        if (!m->graph_exec) {
-            SKN_HIP(ctx, hipStreamSynchronize(ctx->stream));
-            SKN_HIP(ctx, hipStreamBeginCapture(ctx->stream, hipStreamCaptureModeThreadLocal));
-            int rc = decode_step(ctx, m, n_splits);
-            hipGraph_t g = nullptr;
-            hipError_t e = hipStreamEndCapture(ctx->stream, &g);
-            if (rc != SKN_OK) {
-                if (g) (void)hipGraphDestroy(g);
-                return rc;
-            }
-            if (e != hipSuccess) return skn_fail(ctx, SKN_ERR_HIP, "stream capture failed: %s", hipGetErrorString(e));
-            m->graph = g;
-            SKN_HIP(ctx, hipGraphInstantiate(&m->graph_exec, m->graph, nullptr, nullptr, 0));
-            m->graph_splits = n_splits;
-            m->graph_generation = ctx->opt_generation;
-            ctx->stat_captures++;
-        }
-        for (int i = 0; i < n_steps; i++) SKN_HIP(ctx, hipGraphLaunch(m->graph_exec, ctx->stream));
-    }
-    SKN_HIP(ctx, hipMemcpyAsync(tokens_out_host, m->tokens_out, (size_t)n_steps * sizeof(int32_t), hipMemcpyDeviceToHost,
-                                ctx->stream));
-    SKN_HIP(ctx, hipStreamSynchronize(ctx->stream));
+    SKN_TRY(skn_stepper_run(ctx, &m->step, first_token, m->pos, n_steps, n_splits, [&]() { return decode_step(ctx, m, n_splits); },
+                            tokens_out_host));
     m->pos += n_steps;
     for (skn_kv* kv : m->kv) kv->len[0] = m->pos;
     return SKN_OK;

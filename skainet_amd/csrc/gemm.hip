@@ -1980,7 +1980,7 @@ inline size_t align_up(size_t v) { return (v + 255) & ~(size_t)255; }
 
 // Dynamic LDS above 48 KiB must be allowed per kernel and device; done once per context here so that no launch
 // path has to.
-int skn_gemm_init(skn_ctx* ctx) {
+static int skn_gemm_init(skn_ctx* ctx) {
     SKN_HIP(ctx, hipFuncSetAttribute((const void*)gemm_q4k_frag_kernel<2, 2>, hipFuncAttributeMaxDynamicSharedMemorySize, frag_lds_bytes<2, 2>() + 32 * 2 * 2 * 4));
     SKN_HIP(ctx, hipFuncSetAttribute((const void*)gemm_q4k_frag_kernel<2, 1>, hipFuncAttributeMaxDynamicSharedMemorySize, frag_lds_bytes<2, 1>() + 32 * 2 * 1 * 4));
     SKN_HIP(ctx, hipFuncSetAttribute((const void*)gemm_q4k_tall_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, kTlLds));
@@ -1994,6 +1994,7 @@ int skn_gemm_init(skn_ctx* ctx) {
     SKN_HIP(ctx, hipFuncSetAttribute((const void*)gemm_q6k_frag_kernel<4>, hipFuncAttributeMaxDynamicSharedMemorySize, 2 * 4 * 3 * 4096));
     return SKN_OK;
 }
+static skn_family register_family(skn_gemm_init);
 
 int skn_gemm_q4k_multi(skn_ctx* ctx, const skn_gemm_seg* segs, int nseg, int k, const skn_gemm_src& src, int m,
                        bool swiglu_pair) {

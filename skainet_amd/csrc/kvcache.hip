@@ -124,7 +124,8 @@ int skn_kv_advance_len(skn_ctx* ctx, skn_kv* kv, int seq, int n) {
 
 extern "C" {
 
-int skn_kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page_tokens, int max_tokens, skn_kv** out) {
+static int kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page_tokens, int max_tokens, bool shared, int elem_type, int dim,
+                     skn_kv** out) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_create: ctx is null");
     SKN_REQUIRE(ctx, out != nullptr, SKN_ERR_ARG, "skn_kv_create: out is null");
     *out = nullptr;
@@ -136,15 +137,20 @@ int skn_kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page_to
     kv->n_seq = n_seq;
     kv->n_head = n_head;
     kv->head_dim = head_dim;
+    kv->shared = shared;
+    kv->elem_type = elem_type;
+    kv->dim = dim;
     kv->page_tokens = page_tokens;
     kv->max_tokens = max_tokens;
     kv->pages_per_seq = (max_tokens + page_tokens - 1) / page_tokens;
     kv->n_pages = n_seq * kv->pages_per_seq;
     const size_t page_elems = (size_t)n_head * page_tokens * head_dim;
-    const size_t pool_bytes = (size_t)kv->n_pages * page_elems * sizeof(uint16_t);
+    const size_t pool_bytes = (size_t)kv->n_pages * page_elems * (elem_type == SKN_TYPE_F32 ? sizeof(float) : sizeof(uint16_t));
+    const size_t scale_bytes = (size_t)kv->n_pages * page_tokens * sizeof(float);
     const size_t table_bytes = (size_t)n_seq * kv->pages_per_seq * sizeof(int32_t);
     hipError_t e = hipMalloc((void**)&kv->k_pool, pool_bytes);
-    if (e == hipSuccess) e = hipMalloc((void**)&kv->v_pool, pool_bytes);
+    if (e == hipSuccess && !shared) e = hipMalloc((void**)&kv->v_pool, pool_bytes);
+    if (e == hipSuccess && shared) e = hipMalloc((void**)&kv->key_scale, scale_bytes);
     if (e == hipSuccess) e = hipMalloc((void**)&kv->page_table_dev, table_bytes);
     if (e == hipSuccess) e = hipMalloc((void**)&kv->len_dev, (size_t)n_seq * sizeof(int32_t));
     if (e == hipSuccess) e = hipMalloc((void**)&kv->nctx_dev, (size_t)n_seq * sizeof(int32_t));
@@ -163,6 +169,9 @@ int skn_kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page_to
     if (rc == SKN_OK) rc = skn_memset(ctx, kv->len_dev, 0, (size_t)n_seq * sizeof(int32_t));
     if (rc == SKN_OK) rc = skn_memset(ctx, kv->nctx_dev, 0, (size_t)n_seq * sizeof(int32_t));
     if (rc == SKN_OK) rc = skn_memset(ctx, kv->ticket_dev, 0, 16);
+    // (the kernels of a shared cache read its rows up to head_dim: what no token writes is zero)
+    if (rc == SKN_OK && shared) rc = skn_memset(ctx, kv->k_pool, 0, pool_bytes);
+    if (rc == SKN_OK && shared) rc = skn_memset(ctx, kv->key_scale, 0, scale_bytes);
     if (rc != SKN_OK) {
         skn_kv_free(ctx, kv);
         return rc;
@@ -171,12 +180,24 @@ int skn_kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page_to
     return SKN_OK;
 }
 
+int skn_kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page_tokens, int max_tokens, skn_kv** out) {
+    return kv_create(ctx, n_seq, n_head, head_dim, page_tokens, max_tokens, false, SKN_TYPE_F16, head_dim, out);
+}
+
+int skn_kv_create_shared(skn_ctx* ctx, int n_seq, int n_head, int dim, int elem_type, int page_tokens, int max_tokens, skn_kv** out) {
+    SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_create_shared: ctx is null");
+    SKN_REQUIRE(ctx, dim > 0 && dim <= 256, SKN_ERR_SHAPE, "skn_kv_create_shared: heads of %d elements (1 to 256)", dim);
+    SKN_REQUIRE(ctx, elem_type == SKN_TYPE_F16 || elem_type == SKN_TYPE_F32, SKN_ERR_TYPE, "skn_kv_create_shared: type %d (F16 or F32)", elem_type);
+    return kv_create(ctx, n_seq, n_head, dim <= 64 ? 64 : dim <= 128 ? 128 : 256, page_tokens, max_tokens, true, elem_type, dim, out);
+}
+
 int skn_kv_free(skn_ctx* ctx, skn_kv* kv) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_free: ctx is null");
     if (!kv) return SKN_OK;
     (void)hipStreamSynchronize(ctx->stream);
     if (kv->k_pool) (void)hipFree(kv->k_pool);
     if (kv->v_pool) (void)hipFree(kv->v_pool);
+    if (kv->key_scale) (void)hipFree(kv->key_scale);
     if (kv->page_table_dev) (void)hipFree(kv->page_table_dev);
     if (kv->len_dev) (void)hipFree(kv->len_dev);
     if (kv->nctx_dev) (void)hipFree(kv->nctx_dev);
@@ -209,6 +230,7 @@ int skn_kv_append(skn_ctx* ctx, skn_kv* kv, const uint16_t* k_dev, const uint16_
                   int n) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_append: ctx is null");
     SKN_REQUIRE(ctx, kv != nullptr, SKN_ERR_ARG, "skn_kv_append: kv is null");
+    SKN_REQUIRE(ctx, !kv->shared, SKN_ERR_STATE, "skn_kv_append: the cache shares its keys and values");
     SKN_REQUIRE(ctx, n >= 0, SKN_ERR_ARG, "skn_kv_append: negative count");
     if (n == 0) return SKN_OK;
     SKN_REQUIRE(ctx, k_dev && v_dev && seq_ids_host, SKN_ERR_ARG, "skn_kv_append: null pointer");
@@ -250,6 +272,7 @@ int skn_kv_append(skn_ctx* ctx, skn_kv* kv, const uint16_t* k_dev, const uint16_
 int skn_kv_append_run(skn_ctx* ctx, skn_kv* kv, int seq, const uint16_t* k_dev, const uint16_t* v_dev, int n_tokens) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_append_run: ctx is null");
     SKN_REQUIRE(ctx, kv != nullptr, SKN_ERR_ARG, "skn_kv_append_run: kv is null");
+    SKN_REQUIRE(ctx, !kv->shared, SKN_ERR_STATE, "skn_kv_append_run: the cache shares its keys and values");
     SKN_REQUIRE(ctx, seq >= 0 && seq < kv->n_seq, SKN_ERR_RANGE, "skn_kv_append_run: sequence %d of %d", seq, kv->n_seq);
     SKN_REQUIRE(ctx, n_tokens >= 0, SKN_ERR_ARG, "skn_kv_append_run: negative count");
     if (n_tokens == 0) return SKN_OK;
@@ -273,6 +296,7 @@ int skn_kv_append_run(skn_ctx* ctx, skn_kv* kv, int seq, const uint16_t* k_dev, 
 int skn_kv_gather(skn_ctx* ctx, skn_kv* kv, int seq, int t0, int t1, uint16_t* k_out_dev, uint16_t* v_out_dev) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_gather: ctx is null");
     SKN_REQUIRE(ctx, kv != nullptr, SKN_ERR_ARG, "skn_kv_gather: kv is null");
+    SKN_REQUIRE(ctx, !kv->shared, SKN_ERR_STATE, "skn_kv_gather: the cache shares its keys and values");
     SKN_REQUIRE(ctx, seq >= 0 && seq < kv->n_seq, SKN_ERR_RANGE, "skn_kv_gather: sequence %d of %d", seq, kv->n_seq);
     SKN_REQUIRE(ctx, t0 >= 0 && t0 <= t1 && t1 <= kv->len[seq], SKN_ERR_RANGE,
                 "skn_kv_gather: tokens [%d, %d) of a sequence holding %d", t0, t1, kv->len[seq]);

@@ -1866,7 +1866,7 @@ hipError_t allow_big_lds() {
 
 // Dynamic LDS above 48 KiB must be allowed per kernel; done once here so that no launch path (which may run under
 // stream capture) has to.
-int skn_matvec_init(skn_ctx* ctx) {
+static int skn_matvec_init(skn_ctx* ctx) {
     hipError_t (*fns[])() = {allow_big_lds<0, 1>, allow_big_lds<1, 1>, allow_big_lds<2, 1>, allow_big_lds<3, 1>,
                              allow_big_lds<4, 1>, allow_big_lds<0, 2>, allow_big_lds<1, 2>, allow_big_lds<2, 2>,
                              allow_big_lds<3, 2>, allow_big_lds<4, 2>, allow_big_lds<0, 4>, allow_big_lds<1, 4>,
@@ -1931,6 +1931,7 @@ int skn_matvec_init(skn_ctx* ctx) {
 #undef SKN_ALLOW_FUSED
     return SKN_OK;
 }
+static skn_family register_family(skn_matvec_init);
 
 bool skn_matvec_fusable(int ggml_type) {
     return ggml_type == SKN_TYPE_Q4_K || ggml_type == SKN_TYPE_Q5_K || ggml_type == SKN_TYPE_Q4_0 ||

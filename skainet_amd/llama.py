@@ -12,6 +12,7 @@ from dataclasses import dataclass, field
 import numpy as np
 
 from . import runtime, synth
+from .decoder import DecoderModel
 from .runtime import Q4_K, Q6_K, LlamaConfig, LlamaLayer, LlamaWeights
 
 
@@ -100,8 +101,10 @@ def conditioned_weights(cfg: Config, seed: int, gains=None):
     return w
 
 
-class LlamaModel:
+class LlamaModel(DecoderModel):
     """Device-resident model: owns the uploaded weights and the skn_llama handle."""
+
+    PREFIX = "skn_llama"
 
     def __init__(self, ctx: runtime.Context, cfg: Config, weights=None, seed: int = 0, share_layers: bool = False):
         """share_layers=True uploads one layer's weights and points every layer at them (shape-faithful timing
@@ -135,35 +138,6 @@ class LlamaModel:
         h = C.c_void_p()
         ctx._check(ctx.lib.skn_llama_create(ctx.handle, C.byref(c), C.byref(wts), C.byref(h)))
         self.handle = h.value
-
-    def reset(self):
-        self.ctx._check(self.ctx.lib.skn_llama_reset(self.ctx.handle, self.handle))
-
-    def prefill(self, tokens):
-        arr = (C.c_int32 * len(tokens))(*[int(t) for t in tokens])
-        nxt = C.c_int32()
-        self.ctx._check(self.ctx.lib.skn_llama_prefill(self.ctx.handle, self.handle, arr, len(tokens), C.byref(nxt)))
-        return nxt.value
-
-    def decode(self, first_token, n_steps):
-        out = (C.c_int32 * max(n_steps, 1))()
-        self.ctx._check(self.ctx.lib.skn_llama_decode(self.ctx.handle, self.handle, int(first_token), n_steps, out))
-        return list(out[:n_steps])
-
-    def logits(self):
-        p = C.c_void_p()
-        self.ctx._check(self.ctx.lib.skn_llama_logits(self.ctx.handle, self.handle, C.byref(p)))
-        out = np.empty(self.cfg.vocab, dtype=np.float32)
-        self.ctx._check(self.ctx.lib.skn_download(self.ctx.handle, out.ctypes.data, p.value, out.nbytes))
-        return out
-
-    def free(self):
-        if self.handle:
-            self.ctx.lib.skn_llama_free(self.ctx.handle, self.handle)
-            self.handle = None
-        for b in {id(b): b for b in self.bufs.values()}.values():
-            b.free()
-        self.bufs = {}
 
     def weight_bytes_per_token(self):
         """Bytes of weights one decode step streams (embedding row excluded): the HBM floor of a token."""
@@ -265,6 +239,11 @@ def model_from_gguf(ctx: runtime.Context, path: str, max_tokens=None, page_token
         return model
     finally:
         reader.close()
+
+
+def load(ctx: runtime.Context, path: str, dtype=None, max_tokens=None, page_tokens=256) -> LlamaModel:
+    """Loader of the model registry (skainet_amd/models.py); the block formats of the file fix the compute path."""
+    return model_from_gguf(ctx, path, max_tokens, page_tokens)
 
 
 def write_gguf_model(path, cfg: Config, weights):

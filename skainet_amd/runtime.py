@@ -11,6 +11,9 @@ import numpy as np
 
 HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(HERE, "libskainet_hip.so")
+# the part of the library that models with dense (bf16 / fp32) weights need (skainet_amd/build.py); used when the whole
+# library has not been built
+DENSE_LIB_PATH = os.path.join(HERE, "libskainet_dense.so")
 
 F32, F16, Q8_0, Q4_K, Q6_K = 0, 1, 8, 12, 14
 Q4_0, Q4_1, Q5_0, Q5_1, Q2_K, Q5_K, BF16 = 2, 3, 6, 7, 10, 13, 30
@@ -52,6 +55,33 @@ class LlamaWeights(C.Structure):
         ("type_embd", C.c_int32), ("type_head", C.c_int32),
         ("layers", C.POINTER(LlamaLayer)),
     ]
+
+
+class SharedAttn(C.Structure):
+    _fields_ = [
+        ("n_head", C.c_int32), ("scale", C.c_float), ("temp_coef", C.c_float), ("temp_every", C.c_float), ("eps", C.c_float),
+        ("q_norm", C.c_void_p), ("k_norm", C.c_void_p),
+    ]
+
+
+class HybridConfig(C.Structure):
+    _fields_ = [
+        ("n_layer", C.c_int32), ("width", C.c_int32), ("vocab", C.c_int32), ("max_tokens", C.c_int32), ("page_tokens", C.c_int32),
+        ("norm_groups", C.c_int32), ("weight_type", C.c_int32), ("norm_eps", C.c_float), ("residual_mult", C.c_float),
+    ]
+
+
+class HybridLayer(C.Structure):
+    _fields_ = [
+        ("mixer", C.c_int32), ("heads", C.c_int32), ("kv_heads", C.c_int32), ("dim", C.c_int32), ("rank", C.c_int32), ("ff", C.c_int32),
+        ("scale", C.c_float), ("temp_coef", C.c_float), ("temp_every", C.c_float), ("act_pos", C.c_float), ("act_neg", C.c_float),
+        ("norm", C.c_void_p), ("w_in", C.c_void_p), ("b_in", C.c_void_p), ("w_out", C.c_void_p), ("b_out", C.c_void_p),
+        ("q_norm", C.c_void_p), ("k_norm", C.c_void_p), ("w_decay", C.c_void_p), ("b_decay", C.c_void_p), ("o_norm", C.c_void_p),
+    ]
+
+
+class HybridWeights(C.Structure):
+    _fields_ = [("embed", C.c_void_p), ("final_norm", C.c_void_p), ("head", C.c_void_p), ("layers", C.POINTER(HybridLayer))]
 
 
 _SIGNATURES = {
@@ -102,6 +132,14 @@ _SIGNATURES = {
     "skn_attn_decode": (C.c_int, [C.c_void_p, C.c_void_p, C.c_void_p, C.POINTER(C.c_int32), C.c_float, C.c_void_p]),
     "skn_attn_decode_static": (C.c_int, [C.c_void_p, C.c_void_p, C.c_void_p, C.c_float, C.c_void_p]),
     "skn_attn_prefill": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_float, C.c_void_p]),
+    "skn_kv_create_shared": (C.c_int, [C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.POINTER(C.c_void_p)]),
+    "skn_attn_shared": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int, C.POINTER(SharedAttn), C.c_void_p, C.c_void_p, C.c_int, C.c_void_p]),
+    "skn_rstate_create": (C.c_int, [C.c_void_p, C.c_int, C.c_int, C.c_int, C.POINTER(C.c_void_p)]),
+    "skn_rstate_free": (C.c_int, [C.c_void_p, C.c_void_p]),
+    "skn_rstate_reset": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int]),
+    "skn_delta_rule": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p]),
+    "skn_rmsnorm_grouped": (C.c_int, [C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_float, C.c_void_p]),
+    "skn_xielu": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int64, C.c_float, C.c_float, C.c_void_p]),
     "skn_rmsnorm": (C.c_int, [C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_int, C.c_float, C.c_void_p]),
     "skn_rope": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_int, C.c_float]),
     "skn_swiglu": (C.c_int, [C.c_void_p, C.c_void_p, C.c_void_p, C.c_int64, C.c_void_p]),
@@ -116,27 +154,46 @@ _SIGNATURES = {
     "skn_llama_prefill": (C.c_int, [C.c_void_p, C.c_void_p, C.POINTER(C.c_int32), C.c_int, C.POINTER(C.c_int32)]),
     "skn_llama_decode": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int32, C.c_int, C.POINTER(C.c_int32)]),
     "skn_llama_logits": (C.c_int, [C.c_void_p, C.c_void_p, C.POINTER(C.c_void_p)]),
+    "skn_hybrid_create": (C.c_int, [C.c_void_p, C.POINTER(HybridConfig), C.POINTER(HybridWeights), C.POINTER(C.c_void_p)]),
+    "skn_hybrid_free": (C.c_int, [C.c_void_p, C.c_void_p]),
+    "skn_hybrid_reset": (C.c_int, [C.c_void_p, C.c_void_p]),
+    "skn_hybrid_prefill": (C.c_int, [C.c_void_p, C.c_void_p, C.POINTER(C.c_int32), C.c_int, C.POINTER(C.c_int32)]),
+    "skn_hybrid_decode": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int32, C.c_int, C.POINTER(C.c_int32)]),
+    "skn_hybrid_extend": (C.c_int, [C.c_void_p, C.c_void_p, C.POINTER(C.c_int32), C.c_int, C.POINTER(C.c_int32), C.c_int, C.c_void_p]),
+    "skn_hybrid_logits": (C.c_int, [C.c_void_p, C.c_void_p, C.POINTER(C.c_void_p)]),
 }
 
 _LIB = None
 
 
 def load_library():
-    """Loads the in-tree library; raises with the build command when it has not been built."""
+    """Loads the in-tree library; raises with the build command when it has not been built.  Where only the part for dense
+    models has been built, calls outside that part raise."""
     global _LIB
     if _LIB is None:
-        if not os.path.exists(LIB_PATH):
+        path = LIB_PATH if os.path.exists(LIB_PATH) else DENSE_LIB_PATH
+        if not os.path.exists(path):
             raise ImportError(
                 f"{LIB_PATH} is missing: build it with `python -m skainet_amd.build` (needs hipcc); "
                 "there is no CPU fallback for the HIP path"
             )
-        lib = C.CDLL(LIB_PATH)
+        lib = C.CDLL(path)
         for name, (restype, argtypes) in _SIGNATURES.items():
+            if path == DENSE_LIB_PATH and not hasattr(lib, name):
+                setattr(lib, name, _not_built(name))
+                continue
             fn = getattr(lib, name)
             fn.restype = restype
             fn.argtypes = argtypes
         _LIB = lib
     return _LIB
+
+
+def _not_built(name):
+    def fail(*_):
+        raise ImportError(f"{name} is not in {DENSE_LIB_PATH}: build the whole library with `python -m skainet_amd.build`")
+
+    return fail
 
 
 def exported_symbols():
@@ -292,6 +349,63 @@ class KVCache:
             pass
 
 
+class SharedKVCache:
+    """A cache whose values are its keys before their norm (skn_kv_create_shared)."""
+
+    def __init__(self, ctx, n_seq, n_head, dim, page_tokens, max_tokens, elem_type=F16):
+        self.ctx, self.n_head, self.dim = ctx, n_head, dim
+        h = C.c_void_p()
+        ctx._check(ctx.lib.skn_kv_create_shared(ctx.handle, n_seq, n_head, dim, elem_type, page_tokens, max_tokens, C.byref(h)))
+        self.handle = h.value
+
+    def attend(self, seq, params, q, k):
+        """The next tokens of a sequence: host arrays q [n, heads * dim], k [n, n_head * dim] -> [n, heads * dim].  params: dict
+        with n_head, scale, temp_coef, temp_every, eps, q_norm, k_norm."""
+        ctx = self.ctx
+        q, k = (np.ascontiguousarray(a, dtype=np.float32) for a in (q, k))
+        qn, kn = (ctx.to_device(np.ascontiguousarray(params[n], dtype=np.float32)) for n in ("q_norm", "k_norm"))
+        p = SharedAttn(params["n_head"], params["scale"], params.get("temp_coef", 0.0), params.get("temp_every", 0.0), params["eps"], qn.ptr, kn.ptr)
+        qd, kd, out = ctx.to_device(q), ctx.to_device(k), ctx.alloc(q.nbytes)
+        ctx._check(ctx.lib.skn_attn_shared(ctx.handle, self.handle, seq, C.byref(p), qd.ptr, kd.ptr, len(q), out.ptr))
+        return out.download(np.float32, q.size).reshape(q.shape)
+
+    def reset(self, seq=-1):
+        self.ctx._check(self.ctx.lib.skn_kv_reset(self.ctx.handle, self.handle, seq))
+
+    def length(self, seq):
+        return self.ctx.lib.skn_kv_len(self.ctx.handle, self.handle, seq)
+
+    def free(self):
+        if self.handle:
+            self.ctx.lib.skn_kv_free(self.ctx.handle, self.handle)
+            self.handle = None
+
+
+class RecurrentState:
+    """State of generalized delta rule layers (skn_rstate)."""
+
+    def __init__(self, ctx, n_seq, heads, dim):
+        self.ctx, self.heads, self.dim = ctx, heads, dim
+        h = C.c_void_p()
+        ctx._check(ctx.lib.skn_rstate_create(ctx.handle, n_seq, heads, dim, C.byref(h)))
+        self.handle = h.value
+
+    def advance(self, seq, r, k, v, decay, rate):
+        """The next tokens of a sequence: host arrays [n, heads * dim] -> outputs [n, heads * dim]."""
+        bufs = [self.ctx.to_device(np.ascontiguousarray(a, dtype=np.float32)) for a in (r, k, v, decay, rate)]
+        out = self.ctx.alloc(bufs[0].nbytes)
+        self.ctx._check(self.ctx.lib.skn_delta_rule(self.ctx.handle, self.handle, seq, *(b.ptr for b in bufs), len(r), out.ptr))
+        return out.download(np.float32, len(r) * self.heads * self.dim).reshape(len(r), -1)
+
+    def reset(self, seq=-1):
+        self.ctx._check(self.ctx.lib.skn_rstate_reset(self.ctx.handle, self.handle, seq))
+
+    def free(self):
+        if self.handle:
+            self.ctx.lib.skn_rstate_free(self.ctx.handle, self.handle)
+            self.handle = None
+
+
 def _ptr(x):
     if isinstance(x, DeviceBuffer):
         return x.ptr
@@ -416,6 +530,12 @@ class Context:
 
     def rmsnorm(self, x_dev, w_dev, rows, n, eps, y_dev):
         self._check(self.lib.skn_rmsnorm(self.handle, _ptr(x_dev), _ptr(w_dev), rows, n, eps, _ptr(y_dev)))
+
+    def rmsnorm_grouped(self, x_dev, w_dev, rows, n, groups, eps, y_dev):
+        self._check(self.lib.skn_rmsnorm_grouped(self.handle, _ptr(x_dev), _ptr(w_dev), rows, n, groups, eps, _ptr(y_dev)))
+
+    def xielu(self, z_dev, n, pos, neg, out_dev):
+        self._check(self.lib.skn_xielu(self.handle, _ptr(z_dev), n, pos, neg, _ptr(out_dev)))
 
     def rope(self, x_dev, rows, n_head, head_dim, pos0, base):
         self._check(self.lib.skn_rope(self.handle, _ptr(x_dev), rows, n_head, head_dim, pos0, base))
