@@ -5,8 +5,8 @@
 //   out_i = softmax_j <= i ( scale q'_i . k'_j - slope_h (i - j) ) v_j,      slope_h = 2^(-8 (h + 1) / n_head)
 //
 // The cache keeps the projected k (fp16 or fp32) and one factor 1 / rms(k) per token: the norm weights of the key go to the
-// query side (q' . k' = (q' k_norm) . k / rms(k)), so a row serves as key and as value and is read once for both -- and
-// once for all query heads of its group, whose queries a workgroup holds together.
+// query side (q' . k' = (q' k_norm) . k / rms(k)), so a row serves as key and as value and is read once for both.  Where the
+// query heads alone would fill the device several times over, a workgroup takes two of a group at once.
 //
 // Token streams as in csrc/attention.hip: a row is spread over head_dim / 8 lanes, the lanes of a row own a private softmax
 // stream per query head, nothing is staged and no barrier is met while tokens stream.  A step's launch computes the two
@@ -21,7 +21,7 @@ namespace {
 typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 typedef _Float16 half2_t __attribute__((ext_vector_type(2)));
 
-constexpr int kThreads = 512, kWaves = kThreads / 64;
+constexpr int kThreads = 1024, kWaves = kThreads / 64;
 constexpr int kU = 4;           // rows per stream in flight
 constexpr int kMaxSplits = 16;  // what the merge in the output projection's staging is fed at most
 constexpr float kLog2e = 1.4426950408889634f;
@@ -55,7 +55,8 @@ struct Row8<float> {
 };
 
 __device__ __forceinline__ float query_temperature(int pos, float coef, float every) {
-    return coef == 0.f ? 1.f : fmaf(coef, logf((float)floor((double)(pos + 1) / (double)every) + 1.0f), 1.0f);
+    // (the quotient of two integers below 2^24 does not round up to the next one)
+    return coef == 0.f ? 1.f : fmaf(coef, logf(floorf((float)(pos + 1) / every) + 1.0f), 1.0f);
 }
 
 struct AttnArgs {
@@ -63,6 +64,7 @@ struct AttnArgs {
     float* key_scale;
     const int32_t* table;  // the sequence's row of the page table
     int page_tokens, pages_per_seq, n_head, kv_heads, dim;
+    float inv_page;
     float scale_log2e;
     int n_splits;
     float* opart;
@@ -81,18 +83,53 @@ struct AttnArgs {
     float eps, temp_coef, temp_every;
 };
 
-// sum of squares of x[0, n) over the workgroup; red: one float per wavefront (a barrier inside)
-__device__ __forceinline__ void block_sum_squares2(const float* x, int n, const float* y, int m, float* red, float& sx, float& sy) {
-    float a = 0.f, b = 0.f;
-    for (int i = threadIdx.x; i < n; i += blockDim.x) a = fmaf(x[i], x[i], a);
-    for (int i = threadIdx.x; i < m; i += blockDim.x) b = fmaf(y[i], y[i], b);
+// the part of the sum of squares of x[0, n) that this thread has, in two steps so that the first can be issued early: one
+// float4 per thread, then what is left
+__device__ __forceinline__ int whole_quads(const float* x, int n) { return ((uintptr_t)x & 15) == 0 ? n >> 2 : 0; }
+__device__ __forceinline__ float4 first_quad(const float* x, int n) {
+    return (int)threadIdx.x < whole_quads(x, n) ? reinterpret_cast<const float4*>(x)[threadIdx.x] : make_float4(0.f, 0.f, 0.f, 0.f);
+}
+__device__ __forceinline__ float sum_squares(const float4& v, const float* x, int n) {
+    float a = (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+    const int n4 = whole_quads(x, n);
+    for (int i = threadIdx.x + blockDim.x; i < n4; i += blockDim.x) {
+        const float4 w = reinterpret_cast<const float4*>(x)[i];
+        a += (w.x * w.x + w.y * w.y) + (w.z * w.z + w.w * w.w);
+    }
+    for (int i = 4 * n4 + threadIdx.x; i < n; i += blockDim.x) a = fmaf(x[i], x[i], a);
+    return a;
+}
+
+// sums of a and b over the workgroup; red: two floats per wavefront (a barrier inside)
+__device__ __forceinline__ void block_sum2(float& a, float& b, float* red) {
     a = wave_sum(a);
     b = wave_sum(b);
     const int wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
     if ((threadIdx.x & 63) == 0) red[wave] = a, red[nw + wave] = b;
     __syncthreads();
-    sx = sy = 0.f;
-    for (int i = 0; i < nw; i++) sx += red[i], sy += red[nw + i];
+    a = b = 0.f;
+    for (int i = 0; i < nw; i++) a += red[i], b += red[nw + i];
+}
+
+// the value of lane ^ OFF (8, 16 or 32), for sums and maxima over lanes that differ in that bit: f(v, other)
+template <int OFF, typename F>
+__device__ __forceinline__ float with_lane_xor(float v, F f) {
+    if constexpr (OFF == 8) return f(v, __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x128, 0xF, 0xF, true)));  // row rotated by 8
+    else if constexpr (OFF == 16) {
+        const auto r = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+        return f(__uint_as_float(r[0]), __uint_as_float(r[1]));
+    } else {
+        const auto r = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+        return f(__uint_as_float(r[0]), __uint_as_float(r[1]));
+    }
+}
+
+// over the 64 / LPT groups of a wavefront
+template <int LPT, typename F>
+__device__ __forceinline__ float over_groups(float v, F f) {
+    if constexpr (LPT <= 8) v = with_lane_xor<8>(v, f);
+    if constexpr (LPT <= 16) v = with_lane_xor<16>(v, f);
+    return with_lane_xor<32>(v, f);
 }
 
 // grid (splits, kv heads x head groups, query rows)
@@ -102,11 +139,23 @@ __global__ __launch_bounds__(kThreads) void shared_attn_kernel(const AttnArgs p)
     __shared__ float so[kWaves][QG][D];
     __shared__ float sm[kWaves][QG], sl[kWaves][QG];
     __shared__ float red[2 * kWaves];
+    __shared__ __align__(16) float qs[STEP ? QG * D : 4];
     const int split = blockIdx.x, row = blockIdx.z;
     const int per_kv = p.n_head / p.kv_heads, n_groups = (per_kv + QG - 1) / QG;
     const int kvh = blockIdx.y / n_groups, h0 = kvh * per_kv + (blockIdx.y % n_groups) * QG, h_end = (kvh + 1) * per_kv;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int c = lane % LPT, g = lane / LPT, stream = wave * G + g;
+    // what does not wait for the position is requested first: the token's projections, whose norms are computed while the
+    // first cached rows are on their way
+    float4 q4, k4;
+    float q_elem = 0.f;
+    if constexpr (STEP) {
+        static_assert(QG * D <= kThreads, "one element of the group's queries per thread");
+        q4 = first_quad(p.q, p.n_head * p.dim);
+        k4 = first_quad(p.k, p.kv_heads * p.dim);
+        const int i = tid / D, d = tid - i * D, h = min(h0 + i, h_end - 1);
+        if (tid < QG * D && d < p.dim) q_elem = p.q[h * p.dim + d] * p.q_norm[h * p.dim + d] * p.k_norm[kvh * p.dim + d];
+    }
     const int n = STEP ? p.state[2] : p.first_ctx + row;
     const int per = ((n + p.n_splits - 1) / p.n_splits + NS - 1) / NS * NS;
     const int t_begin = split * per, t_end = min(n, t_begin + per);
@@ -120,7 +169,7 @@ __global__ __launch_bounds__(kThreads) void shared_attn_kernel(const AttnArgs p)
 #pragma unroll
         for (int u = 0; u < U; u++) {
             const int t = max(min(base + u * NS + stream, t_end - 1), 0);  // past the end: a valid row, masked below
-            const int pi = t / p.page_tokens, slot = t - pi * p.page_tokens;
+            const int pi = (int)(((float)t + 0.5f) * p.inv_page), slot = t - pi * p.page_tokens;  // (exact below 2^22 tokens)
             int page = __shfl(my_page, pi & 63, 64);
             if (pi >= 64) page = p.table[pi];
             rows[u].load(pool + (((int64_t)page * p.kv_heads + kvh) * p.page_tokens + slot) * D + c * 8);
@@ -131,8 +180,9 @@ __global__ __launch_bounds__(kThreads) void shared_attn_kernel(const AttnArgs p)
 
     float qf[QG][8], fq = p.scale_log2e, newest_scale = 0.f;
     if constexpr (STEP) {
-        float sq, sk;
-        block_sum_squares2(p.q, p.n_head * p.dim, p.k, p.kv_heads * p.dim, red, sq, sk);
+        if (tid < QG * D) qs[tid] = q_elem;  // (the barrier of the sums covers it)
+        float sq = sum_squares(q4, p.q, p.n_head * p.dim), sk = sum_squares(k4, p.k, p.kv_heads * p.dim);
+        block_sum2(sq, sk, red);
         newest_scale = 1.0f / sqrtf(sk / (float)(p.kv_heads * p.dim) + p.eps);
         fq *= query_temperature(n - 1, p.temp_coef, p.temp_every) / sqrtf(sq / (float)(p.n_head * p.dim) + p.eps);
         if (split == 0 && blockIdx.y == 0 && tid == 0) {  // for the steps to come (this one uses its own)
@@ -141,13 +191,8 @@ __global__ __launch_bounds__(kThreads) void shared_attn_kernel(const AttnArgs p)
         }
 #pragma unroll
         for (int i = 0; i < QG; i++) {
-            const int h = min(h0 + i, h_end - 1);
-#pragma unroll
-            for (int j = 0; j < 8; j++) {
-                const int d = c * 8 + j, at = min(d, p.dim - 1);
-                const float v = p.q[h * p.dim + at] * p.q_norm[h * p.dim + at] * p.k_norm[kvh * p.dim + at];
-                qf[i][j] = d < p.dim ? v : 0.f;
-            }
+            const float4 a = *reinterpret_cast<const float4*>(&qs[i * D + c * 8]), b = *reinterpret_cast<const float4*>(&qs[i * D + c * 8 + 4]);
+            qf[i][0] = a.x, qf[i][1] = a.y, qf[i][2] = a.z, qf[i][3] = a.w, qf[i][4] = b.x, qf[i][5] = b.y, qf[i][6] = b.z, qf[i][7] = b.w;
         }
     } else {
 #pragma unroll
@@ -192,10 +237,10 @@ __global__ __launch_bounds__(kThreads) void shared_attn_kernel(const AttnArgs p)
 #pragma unroll
             for (int u = 0; u < U; u++) m_new = fmaxf(m_new, sc[i][u]);
             const float m_safe = m_new == -INFINITY ? 0.f : m_new;  // keeps exp2(-inf - -inf) out of the arithmetic
-            const float alpha = exp2f(m_run[i] - m_safe);
+            const float alpha = __builtin_amdgcn_exp2f(m_run[i] - m_safe);
             float sum = 0.f;
 #pragma unroll
-            for (int u = 0; u < U; u++) sum += pr[i][u] = exp2f(sc[i][u] - m_safe);
+            for (int u = 0; u < U; u++) sum += pr[i][u] = __builtin_amdgcn_exp2f(sc[i][u] - m_safe);
             l_run[i] = fmaf(l_run[i], alpha, sum);
             m_run[i] = m_new;
 #pragma unroll
@@ -211,29 +256,22 @@ __global__ __launch_bounds__(kThreads) void shared_attn_kernel(const AttnArgs p)
                 for (int j = 0; j < 8; j++) o[i][j] = fmaf(pr[i][u], vf[j], o[i][j]);
         }
     };
-    for (int base = t_begin; base < t_end; base += 2 * NS * U) {
+    for (int base = t_begin; base < t_end; base += NS * U) {
         fetch(nxt, cs_nxt, base + NS * U);
         absorb(cur, cs_cur, base);
-        fetch(cur, cs_cur, base + 2 * NS * U);
-        absorb(nxt, cs_nxt, base + NS * U);
+#pragma unroll
+        for (int u = 0; u < U; u++) cur[u] = nxt[u], cs_cur[u] = cs_nxt[u];
     }
 
     // the G streams of the wavefront (lanes with the same c hold the same elements), then the wavefronts through LDS
 #pragma unroll
     for (int i = 0; i < QG; i++) {
-        float mw = m_run[i];
+        const auto add = [](float a, float b) { return a + b; };
+        const float mw = over_groups<LPT>(m_run[i], [](float a, float b) { return fmaxf(a, b); });
+        const float w = __builtin_amdgcn_exp2f(m_run[i] - (mw == -INFINITY ? 0.f : mw));  // (an empty stream: exp2(-inf) = 0)
+        const float lw = over_groups<LPT>(l_run[i] * w, add);
 #pragma unroll
-        for (int off = LPT; off < 64; off <<= 1) mw = fmaxf(mw, __shfl_xor(mw, off, 64));
-        const float w = exp2f(m_run[i] - (mw == -INFINITY ? 0.f : mw));  // (an empty stream: exp2(-inf) = 0)
-        float lw = l_run[i] * w;
-#pragma unroll
-        for (int j = 0; j < 8; j++) o[i][j] *= w;
-#pragma unroll
-        for (int off = LPT; off < 64; off <<= 1) {
-            lw += __shfl_xor(lw, off, 64);
-#pragma unroll
-            for (int j = 0; j < 8; j++) o[i][j] += __shfl_xor(o[i][j], off, 64);
-        }
+        for (int j = 0; j < 8; j++) o[i][j] = over_groups<LPT>(o[i][j] * w, add);
         if (g == 0) {
 #pragma unroll
             for (int j = 0; j < 8; j++) so[wave][i][c * 8 + j] = o[i][j];
@@ -250,7 +288,7 @@ __global__ __launch_bounds__(kThreads) void shared_attn_kernel(const AttnArgs p)
         const float m_safe = m == -INFINITY ? 0.f : m;
 #pragma unroll
         for (int w = 0; w < kWaves; w++) {
-            const float f = exp2f(sm[w][i] - m_safe);
+            const float f = __builtin_amdgcn_exp2f(sm[w][i] - m_safe);
             acc = fmaf(f, so[w][i][d], acc);
             l = fmaf(f, sl[w][i], l);
         }
@@ -277,8 +315,8 @@ __global__ __launch_bounds__(256) void shared_prep_kernel(const float* __restric
     const int row = blockIdx.x, pos = pos0 + row;
     const float* qr = q + (int64_t)row * ldq;
     const float* kr = k + (int64_t)row * ldk;
-    float sq, sk;
-    block_sum_squares2(qr, n_head * dim, kr, kv_heads * dim, red, sq, sk);
+    float sq = sum_squares(first_quad(qr, n_head * dim), qr, n_head * dim), sk = sum_squares(first_quad(kr, kv_heads * dim), kr, kv_heads * dim);
+    block_sum2(sq, sk, red);
     const float rk = 1.0f / sqrtf(sk / (float)(kv_heads * dim) + eps);
     const float rq = query_temperature(pos, temp_coef, temp_every) / sqrtf(sq / (float)(n_head * dim) + eps);
     const int page = table[pos / page_tokens], slot = pos % page_tokens, per_kv = n_head / kv_heads;
@@ -296,25 +334,36 @@ __global__ __launch_bounds__(256) void shared_prep_kernel(const float* __restric
     }
 }
 
-template <typename E, int D, bool STEP>
-int launch_qg(skn_ctx* ctx, const AttnArgs& a, int rows) {
+// query heads a workgroup of a step takes: as few as keep the workgroups within two per compute unit
+int heads_per_group(const skn_ctx* ctx, int per_kv, int kv_heads, int splits) {
+    int qg = 1;
+    while (qg < 2 && qg * 2 <= per_kv && splits * kv_heads * ((per_kv + qg - 1) / qg) > 2 * ctx->compute_units) qg *= 2;
+    return qg;
+}
+
+template <typename E, int D, int QG, bool STEP>
+int launch_as(skn_ctx* ctx, const AttnArgs& a, int rows) {
     const int per_kv = a.n_head / a.kv_heads;
-    auto grid = [&](int qg) { return dim3(a.n_splits, a.kv_heads * ((per_kv + qg - 1) / qg), rows); };
-    if (per_kv == 1) skn_launch(ctx, shared_attn_kernel<E, D, 1, STEP>, grid(1), dim3(kThreads), 0, a);
-    else if (per_kv == 2) skn_launch(ctx, shared_attn_kernel<E, D, 2, STEP>, grid(2), dim3(kThreads), 0, a);
-    else skn_launch(ctx, shared_attn_kernel<E, D, 4, STEP>, grid(4), dim3(kThreads), 0, a);
+    skn_launch(ctx, shared_attn_kernel<E, D, QG, STEP>, dim3(a.n_splits, a.kv_heads * ((per_kv + QG - 1) / QG), rows), dim3(kThreads), 0, a);
     SKN_LAUNCH_CHECK(ctx);
     return SKN_OK;
 }
 
+template <int D, bool STEP>
+int launch_dim(skn_ctx* ctx, const skn_kv* kv, const AttnArgs& a, int rows) {
+    if (kv->elem_type == SKN_TYPE_F32) return launch_as<float, D, 1, STEP>(ctx, a, rows);
+    if constexpr (STEP) {
+        const int qg = heads_per_group(ctx, a.n_head / a.kv_heads, a.kv_heads, a.n_splits);
+        if (qg == 2) return launch_as<uint16_t, D, 2, true>(ctx, a, rows);
+    }
+    return launch_as<uint16_t, D, 1, STEP>(ctx, a, rows);
+}
+
 template <bool STEP>
 int launch_attn(skn_ctx* ctx, const skn_kv* kv, const AttnArgs& a, int rows) {
-    const bool f32 = kv->elem_type == SKN_TYPE_F32;
-    switch (kv->head_dim) {
-        case 64: return f32 ? launch_qg<float, 64, STEP>(ctx, a, rows) : launch_qg<uint16_t, 64, STEP>(ctx, a, rows);
-        case 128: return f32 ? launch_qg<float, 128, STEP>(ctx, a, rows) : launch_qg<uint16_t, 128, STEP>(ctx, a, rows);
-        default: return f32 ? launch_qg<float, 256, STEP>(ctx, a, rows) : launch_qg<uint16_t, 256, STEP>(ctx, a, rows);
-    }
+    if (kv->head_dim == 64) return launch_dim<64, STEP>(ctx, kv, a, rows);
+    if (kv->head_dim == 128) return launch_dim<128, STEP>(ctx, kv, a, rows);
+    return launch_dim<256, STEP>(ctx, kv, a, rows);
 }
 
 AttnArgs base_args(const skn_kv* kv, int seq, const skn_shared_attn& p) {
@@ -324,6 +373,7 @@ AttnArgs base_args(const skn_kv* kv, int seq, const skn_shared_attn& p) {
     a.table = kv->page_table_dev + (size_t)seq * kv->pages_per_seq;
     a.page_tokens = kv->page_tokens;
     a.pages_per_seq = kv->pages_per_seq;
+    a.inv_page = 1.0f / (float)kv->page_tokens;
     a.n_head = p.n_head;
     a.kv_heads = kv->n_head;
     a.dim = kv->dim;
@@ -395,13 +445,13 @@ int skn_shared_attn_step(skn_ctx* ctx, skn_kv* kv, int seq, const skn_shared_att
     return launch_attn<true>(ctx, kv, a, 1);
 }
 
-// Splits for contexts up to max_ctx: a power of two, so that a workgroup has at least two rounds of requests and the
-// workgroups do not outnumber the compute units (the merge reads every split in every workgroup that follows).
+// Splits for contexts up to max_ctx: a power of two, at most eight (sixteen where few heads would read a long context: the
+// merge reads every split in every workgroup that follows), so that a workgroup has at least a round of requests.
 int skn_shared_attn_splits(skn_ctx* ctx, const skn_kv* kv, int n_head, int max_ctx) {
-    const int per_kv = n_head / kv->n_head, qg = per_kv >= 4 ? 4 : per_kv >= 2 ? 2 : 1;
-    const int wgs = kv->n_head * ((per_kv + qg - 1) / qg), round = kWaves * 512 / kv->head_dim * kU;
+    const int round = kWaves * 512 / kv->head_dim * kU;
+    const int most = n_head * 8 <= ctx->compute_units / 2 ? kMaxSplits : 8;
     int n = 1;
-    while (n < kMaxSplits && n * round < max_ctx && 2 * n * wgs <= ctx->compute_units) n *= 2;
+    while (n < most && n * round < max_ctx) n *= 2;
     return n;
 }
 

@@ -5,10 +5,12 @@
 // the L lanes by DPP, and the state never leaves the registers between two tokens.  Because u = k / |k|, the removal term
 // is (a k / |k|^2) (k^T S): one vector b = a k / (sum k^2 + 1e-6) beside k serves it.
 //
-// Prompts take two launches.  delta_pack_kernel writes, per head and token, the five vectors k, w, b, r, v one after the other, padded to
-// the lanes' channels; delta_scan_kernel -- one small workgroup per head and run of columns -- copies sixteen tokens at a
-// time of that stream straight into LDS, one block ahead of the tokens it computes, and reads each token's vectors one
-// token ahead.  The tokens of a sequence are a chain; what is parallel are the heads and the columns.
+// Prompts take two launches.  delta_pack_kernel writes, per head and token, the five vectors k, w, b, r, v one after the
+// other, padded to the lanes' channels (and tokens that change nothing up to whole blocks); delta_scan_kernel -- one small
+// workgroup per head and run of columns -- has the next 20 KB block of that stream on its way into registers while it computes
+// the tokens of the current one out of LDS, each token's vectors read one token ahead.  (Copied straight into LDS instead,
+// the compiler puts a wait for the copy in front of the next LDS read.)  The tokens of a sequence are a chain; what is
+// parallel are the heads and the columns.
 // A decode step is one launch, one workgroup per head: the decay's low-rank product, the step, the head's norm and the gate.
 #include "dense.h"
 #include "rstate.h"
@@ -50,14 +52,20 @@ __device__ __forceinline__ float delta_column(Vec8& s, const Vec8& k, const Vec8
 
 constexpr int kVecs = 5;  // k, w, b, r, v
 
-// one wavefront per (token, head)
+constexpr int kBlockFloats = kVecs * 1024;  // a block of the packed stream: 1024 / dim_pad tokens
+constexpr int kTrash = 64;                  // floats behind the stream that lanes without a column store to
+
+__host__ __device__ inline int block_tokens(int dim_pad) { return 1024 / dim_pad; }
+__host__ __device__ inline int padded_tokens(int n, int dim_pad) { return (n + block_tokens(dim_pad) - 1) / block_tokens(dim_pad) * block_tokens(dim_pad); }
+
+// one wavefront per (token, head); n_pad: tokens with those that only fill the last block (k = b = 0, w = 1)
 __global__ __launch_bounds__(256) void delta_pack_kernel(const float* __restrict__ r, const float* __restrict__ k, const float* __restrict__ v,
-                                                         const float* __restrict__ w, const float* __restrict__ a, int ld, int n, int heads, int dim,
-                                                         int dim_pad, float* __restrict__ pack) {
+                                                         const float* __restrict__ w, const float* __restrict__ a, int ld, int n, int n_pad, int heads,
+                                                         int dim, int dim_pad, float* __restrict__ pack) {
     const int id = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    if (id >= n * heads) return;
+    if (id >= n_pad * heads) return;
     const int t = id / heads, h = id - t * heads;
-    const int64_t at = (int64_t)t * ld + h * dim;
+    const int64_t at = (int64_t)min(t, n - 1) * ld + h * dim;
     float kk[4], ss = 0.f;
 #pragma unroll
     for (int i = 0; i < 4; i++) {
@@ -66,36 +74,28 @@ __global__ __launch_bounds__(256) void delta_pack_kernel(const float* __restrict
         ss = fmaf(kk[i], kk[i], ss);
     }
     const float inv = 1.0f / (wave_sum(ss) + kUnitEps);
-    float* out = pack + ((int64_t)h * n + t) * kVecs * dim_pad;
+    float* out = pack + ((int64_t)h * n_pad + t) * kVecs * dim_pad;
 #pragma unroll
     for (int i = 0; i < 4; i++) {
         const int d = lane + 64 * i;
         if (d >= dim_pad) continue;
-        const bool in = d < dim;
-        out[d] = kk[i];
-        out[dim_pad + d] = in ? w[at + d] : 0.f;
+        const bool in = d < dim && t < n;
+        out[d] = in ? kk[i] : 0.f;
+        out[dim_pad + d] = in ? w[at + d] : 1.f;
         out[2 * dim_pad + d] = in ? a[at + d] * kk[i] * inv : 0.f;
         out[3 * dim_pad + d] = in ? r[at + d] : 0.f;
         out[4 * dim_pad + d] = in ? v[at + d] : 0.f;
     }
 }
 
-template <int L>
-constexpr int scan_block_tokens() {
-    return L >= 32 ? 8 : 16;
-}
-template <int L>
-constexpr int scan_lds_bytes() {
-    return 2 * scan_block_tokens<L>() * kVecs * L * 8 * 4;
-}
-
 // grid (column runs, heads); NW wavefronts of 64 / L columns each
 template <int L, int NW>
-__global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __restrict__ pack, int n, int heads, int dim, float* __restrict__ state,
-                                                             float* __restrict__ o) {
-    extern __shared__ __align__(16) float lds[];
-    constexpr int DP = 8 * L, C = scan_block_tokens<L>(), kBlock = C * kVecs * DP, kReq = kBlock * 4 / 1024;
-    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), h = blockIdx.y;
+__global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __restrict__ pack, int n, int n_pad, int heads, int dim,
+                                                             float* __restrict__ state, float* __restrict__ o, float* __restrict__ trash) {
+    __shared__ __align__(16) float lds[2][kBlockFloats];
+    constexpr int DP = 8 * L, C = 1024 / DP, kTurns = kBlockFloats / 4 / (64 * NW);  // float4 per thread and block
+    static_assert(kTurns * 4 * 64 * NW == kBlockFloats, "a block is whole float4 per thread");
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.y;
     const int rl = lane & (L - 1);
     const int col = (blockIdx.x * NW + wave) * (64 / L) + lane / L;
     const bool live = col < dim;
@@ -103,44 +103,56 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
     float* sp = state + ((int64_t)h * dim + colc) * DP + 8 * rl;
     Vec8 s;
     s.load(sp);
-    const uint8_t* src = (const uint8_t*)(pack + (int64_t)h * n * kVecs * DP);
-    const int64_t last = (int64_t)n * kVecs * DP * 4 - 16;  // (past the end: the last piece again, not used)
-    auto request = [&](int blk) __attribute__((always_inline)) {
-        const int64_t at = (int64_t)blk * kBlock * 4;
-        for (int i = wave; i < kReq; i += NW)
-            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + min(at + i * 1024 + lane * 16, last)),
-                                             (__attribute__((address_space(3))) void*)((uint8_t*)lds + (blk & 1) * kBlock * 4 + i * 1024), 16, 0, 0);
-    };
-    const int blocks = (n + C - 1) / C;
-    request(0);
-    float keep = 0.f;
-    for (int blk = 0; blk < blocks; blk++) {
-        asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
-        if (blk + 1 < blocks) request(blk + 1);
-        const float* base = lds + (blk & 1) * kBlock;
-        const int t0 = blk * C, count = min(C, n - t0);
+    const float4* src = reinterpret_cast<const float4*>(pack + (int64_t)h * n_pad * kVecs * DP) + tid;
+    const int blocks = n_pad / C;
+    float4 ahead[kTurns];
+#pragma unroll
+    for (int i = 0; i < kTurns; i++) ahead[i] = src[i * 64 * NW];
+
+    struct Token {
         Vec8 k, w, b, r;
         float v;
-        auto read = [&](int t) __attribute__((always_inline)) {
+    };
+    for (int blk = 0; blk < blocks; blk++) {
+        // (this buffer was last read two blocks ago, and everyone has passed the barrier since)
+        float4* dst = reinterpret_cast<float4*>(lds[blk & 1]) + tid;
+#pragma unroll
+        for (int i = 0; i < kTurns; i++) dst[i * 64 * NW] = ahead[i];
+        const float4* next = src + (int64_t)min(blk + 1, blocks - 1) * (kBlockFloats / 4);
+#pragma unroll
+        for (int i = 0; i < kTurns; i++) ahead[i] = next[i * 64 * NW];
+        __builtin_amdgcn_sched_barrier(0);
+        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+        const float* base = lds[blk & 1];
+        const int t0 = blk * C;
+        auto read = [&](Token& x, int t) __attribute__((always_inline)) {
             const float* p = base + t * kVecs * DP;
-            k.load(p + 8 * rl);
-            w.load(p + DP + 8 * rl);
-            b.load(p + 2 * DP + 8 * rl);
-            r.load(p + 3 * DP + 8 * rl);
-            v = p[4 * DP + colc];
+            x.k.load(p + 8 * rl);
+            x.w.load(p + DP + 8 * rl);
+            x.b.load(p + 2 * DP + 8 * rl);
+            x.r.load(p + 3 * DP + 8 * rl);
+            x.v = p[4 * DP + colc];
         };
-        read(0);
-        for (int t = 0; t < count; t++) {
-            const Vec8 k1 = k, w1 = w, b1 = b, r1 = r;
-            const float v1 = v;
-            read(min(t + 1, C - 1));
-            const float out = delta_column<L>(s, k1, w1, b1, r1, v1);
-            // the L lanes of a column keep the outputs of L consecutive tokens and store them together
-            const int tt = t0 + t;
-            if ((tt & (L - 1)) == rl) keep = out;
-            if ((tt & (L - 1)) == L - 1 || tt == n - 1) {
-                const int mine = (tt & ~(L - 1)) + rl;
-                if (live && mine <= tt) o[((int64_t)mine * heads + h) * dim + col] = keep;
+        Token even, odd;
+        read(even, 0);
+        constexpr int G = L < C ? L : C;  // the L lanes of a column keep the outputs of G tokens and store them together
+        float keep = 0.f;
+#pragma unroll
+        for (int t = 0; t < C; t += 2) {
+            read(odd, t + 1);
+            __builtin_amdgcn_sched_barrier(0);
+            const float o0 = delta_column<L>(s, even.k, even.w, even.b, even.r, even.v);
+            keep = rl == t % G ? o0 : keep;
+            if (t + 2 < C) read(even, t + 2);
+            __builtin_amdgcn_sched_barrier(0);
+            const float o1 = delta_column<L>(s, odd.k, odd.w, odd.b, odd.r, odd.v);
+            keep = rl == t % G + 1 ? o1 : keep;
+            if ((t + 2) % G == 0) {
+                // (one store whatever the lane: a skipped one would leave the number of requests outstanding unknown, and
+                // the wait for the next block would wait for every store)
+                const int mine = t0 + t + 2 - G + rl;
+                float* p = live && rl < G && mine < n ? o + ((int64_t)mine * heads + h) * dim + col : trash + lane;
+                *p = keep;
             }
         }
     }
@@ -253,9 +265,10 @@ __global__ __launch_bounds__(64 * NW) void delta_step_kernel(const skn_delta_ste
 
 template <int L, int NW>
 int launch_scan(skn_ctx* ctx, const skn_rstate* st, const float* pack, int n, float* state, float* o) {
-    const int per_wg = NW * (64 / L);
-    skn_launch(ctx, delta_scan_kernel<L, NW>, dim3((st->dim + per_wg - 1) / per_wg, st->heads), dim3(64 * NW), (size_t)scan_lds_bytes<L>(), pack, n,
-               st->heads, st->dim, state, o);
+    const int per_wg = NW * (64 / L), n_pad = padded_tokens(n, st->dim_pad);
+    float* trash = const_cast<float*>(pack) + (size_t)n_pad * st->heads * kVecs * st->dim_pad;
+    skn_launch(ctx, delta_scan_kernel<L, NW>, dim3((st->dim + per_wg - 1) / per_wg, st->heads), dim3(64 * NW), 0, pack, n, n_pad, st->heads, st->dim, state,
+               o, trash);
     SKN_LAUNCH_CHECK(ctx);
     return SKN_OK;
 }
@@ -278,23 +291,6 @@ int scan_waves(skn_ctx* ctx, const skn_rstate* st, const float* pack, int n, flo
     return launch_scan<L, 1>(ctx, st, pack, n, state, o);
 }
 
-template <int L, int NW>
-int allow_scan(skn_ctx* ctx) {
-    SKN_HIP(ctx, hipFuncSetAttribute((const void*)delta_scan_kernel<L, NW>, hipFuncAttributeMaxDynamicSharedMemorySize, scan_lds_bytes<L>()));
-    return SKN_OK;
-}
-
-int delta_init(skn_ctx* ctx) {
-    SKN_TRY((allow_scan<16, 1>(ctx)));
-    SKN_TRY((allow_scan<16, 2>(ctx)));
-    SKN_TRY((allow_scan<16, 4>(ctx)));
-    SKN_TRY((allow_scan<32, 1>(ctx)));
-    SKN_TRY((allow_scan<32, 2>(ctx)));
-    SKN_TRY((allow_scan<32, 4>(ctx)));
-    return SKN_OK;
-}
-skn_family register_family(delta_init);
-
 __global__ void fill_zero_kernel(float4* p, int64_t n) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i < n) p[i] = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -302,13 +298,16 @@ __global__ void fill_zero_kernel(float4* p, int64_t n) {
 
 }  // namespace
 
-size_t skn_delta_pack_floats(const skn_rstate* st, int n) { return (size_t)n * st->heads * kVecs * st->dim_pad; }
+size_t skn_delta_pack_floats(const skn_rstate* st, int n) {
+    return (size_t)padded_tokens(n, st->dim_pad) * st->heads * kVecs * st->dim_pad + kTrash;
+}
 
 int skn_delta_rows(skn_ctx* ctx, skn_rstate* st, int seq, const float* r, const float* k, const float* v, const float* w, const float* a, int ld, int n,
                    float* pack, float* o) {
-    SKN_REQUIRE(ctx, n > 0 && (int64_t)n * st->heads < ((int64_t)1 << 31) - 4, SKN_ERR_SHAPE, "delta rule: %d tokens x %d heads", n, st->heads);
-    skn_launch(ctx, delta_pack_kernel, dim3((unsigned)(((int64_t)n * st->heads + 3) / 4)), dim3(256), 0, r, k, v, w, a, ld, n, st->heads, st->dim, st->dim_pad,
-               pack);
+    SKN_REQUIRE(ctx, n > 0 && (int64_t)(n + 32) * st->heads < ((int64_t)1 << 31) - 4, SKN_ERR_SHAPE, "delta rule: %d tokens x %d heads", n, st->heads);
+    const int n_pad = padded_tokens(n, st->dim_pad);
+    skn_launch(ctx, delta_pack_kernel, dim3((unsigned)(((int64_t)n_pad * st->heads + 3) / 4)), dim3(256), 0, r, k, v, w, a, ld, n, n_pad, st->heads, st->dim,
+               st->dim_pad, pack);
     SKN_LAUNCH_CHECK(ctx);
     float* s = st->seq_state(seq);
     switch (st->dim_pad) {

@@ -3,8 +3,8 @@
 // The input is staged once per workgroup in LDS -- plain, divided group by group by its root mean square (the norm ahead
 // of a layer), or with the split partials of an attention merged on the way in -- as two planes of float4 (even and odd
 // fours of elements), so that the eight activations of a 16-byte piece of bf16 weights are two conflict-free 16-byte
-// reads.  A wavefront owns two rows at a time and walks on through the stacked rows; the weights of its next few
-// requests are under way while it multiplies, the first ones from before the staging.  Epilogue: bias and the operation
+// reads.  A wavefront takes a row at a time and walks on through the stacked rows; its next requests are under way while it
+// multiplies, the first ones from before the staging.  Epilogue: bias and the operation
 // of the segment, or the residual sum; a key projection also goes to its page of the cache.
 #include "dense.h"
 
@@ -15,10 +15,10 @@ namespace {
 
 typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 
-constexpr int kThreads = 512, kWaves = kThreads / 64;
-constexpr int kR = 2;  // rows per wavefront and turn
-constexpr int kU = 4;  // 16-byte pieces per row and lane in flight
-constexpr int kMaxGroups = 256, kMaxMerge = 2048;  // norm groups; heads x splits of a merge
+constexpr int kThreads = 1024, kWaves = kThreads / 64;
+constexpr int kR = 1;  // rows per wavefront and turn (measured with two as well: slower at 1024 threads)
+constexpr int kU = 4;  // 16-byte pieces per row and lane in flight, twice
+constexpr int kMaxGroups = 256, kMaxMerge = 4096, kMaxSplits = 16;  // norm groups; heads x splits and splits of a merge
 
 struct XPlanes {
     float4* even;
@@ -83,26 +83,39 @@ __device__ __forceinline__ void stage_group_norm(const skn_matvec_src& s, const 
 __device__ __forceinline__ void stage_merge(const skn_matvec_src& s, const XPlanes& xs, float* red) {
     const int tid = threadIdx.x;
     for (int h = tid; h < s.heads; h += kThreads) {
+        float2 ml[kMaxSplits];  // (all requested before the first is used)
+#pragma unroll
+        for (int i = 0; i < kMaxSplits; i++) ml[i] = reinterpret_cast<const float2*>(s.ml)[min(i, s.splits - 1) * s.heads + h];
         float m = -INFINITY, l = 0.f;
-        for (int i = 0; i < s.splits; i++) m = fmaxf(m, s.ml[2 * (i * s.heads + h)]);
-        for (int i = 0; i < s.splits; i++) {
-            const float f = exp2f(s.ml[2 * (i * s.heads + h)] - m);  // (an empty split: exp2(-inf) = 0)
-            l = fmaf(f, s.ml[2 * (i * s.heads + h) + 1], l);
-            red[h * s.splits + i] = f;
+#pragma unroll
+        for (int i = 0; i < kMaxSplits; i++) m = fmaxf(m, ml[i].x);
+#pragma unroll
+        for (int i = 0; i < kMaxSplits; i++) {
+            ml[i].x = i < s.splits ? __builtin_amdgcn_exp2f(ml[i].x - m) : 0.f;  // (an empty split: exp2(-inf) = 0)
+            l = fmaf(ml[i].x, ml[i].y, l);
         }
         const float inv = 1.0f / l;
-        for (int i = 0; i < s.splits; i++) red[h * s.splits + i] *= inv;
+#pragma unroll
+        for (int i = 0; i < kMaxSplits; i++)
+            if (i < s.splits) red[h * s.splits + i] = ml[i].x * inv;
     }
     __syncthreads();
     if ((s.dim & 3) == 0) {
         const int dq = s.dim >> 2;
+        const int64_t step = (int64_t)s.heads * s.dim_pad;
         for (int q = tid; q < s.heads * dq; q += kThreads) {
             const int h = q / dq, c = q - h * dq;
+            const float* p = s.x0 + (int64_t)h * s.dim_pad + 4 * c;
             float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
-            for (int i = 0; i < s.splits; i++) {
-                const float f = red[h * s.splits + i];
-                const float4 v = *reinterpret_cast<const float4*>(s.x0 + ((int64_t)i * s.heads + h) * s.dim_pad + 4 * c);
-                a.x = fmaf(f, v.x, a.x), a.y = fmaf(f, v.y, a.y), a.z = fmaf(f, v.z, a.z), a.w = fmaf(f, v.w, a.w);
+            for (int i0 = 0; i0 < s.splits; i0 += 8) {
+                float4 v[8];
+#pragma unroll
+                for (int i = 0; i < 8; i++) v[i] = *reinterpret_cast<const float4*>(p + min(i0 + i, s.splits - 1) * step);
+#pragma unroll
+                for (int i = 0; i < 8; i++) {
+                    const float f = i0 + i < s.splits ? red[h * s.splits + i0 + i] : 0.f;
+                    a.x = fmaf(f, v[i].x, a.x), a.y = fmaf(f, v[i].y, a.y), a.z = fmaf(f, v[i].z, a.z), a.w = fmaf(f, v[i].w, a.w);
+                }
             }
             xs.quad(q) = a;
         }
@@ -262,13 +275,11 @@ int launch(skn_ctx* ctx, const skn_dense_mat& w, const skn_matvec_src& src, cons
     constexpr int V = 16 / (int)sizeof(W);
     const int chunk = 64 * kU * V;  // elements of a turn: the planes hold whole turns
     const int plane = (w.k_pad + chunk - 1) / chunk * chunk / 8;
-    const size_t scratch = MODE == SKN_XSRC_GROUP_NORM ? (kMaxGroups + 16) * 4 : MODE == SKN_XSRC_MERGE ? (size_t)src.heads * src.splits * 4 : 0;
+    const size_t scratch = MODE == SKN_XSRC_GROUP_NORM ? (kMaxGroups + 16 * kWaves) * 4 : MODE == SKN_XSRC_MERGE ? (size_t)src.heads * src.splits * 4 : 0;
     const size_t lds = (size_t)plane * 32 + scratch;
     SKN_REQUIRE(ctx, lds <= kMaxLds, SKN_ERR_SHAPE, "dense matvec: %d columns need %zu bytes of LDS (at most %d)", w.k_pad, lds, kMaxLds);
-    const int groups = (w.rows + kR - 1) / kR;
-    // as many workgroups as are resident at once: the staging of one serves all the rows its wavefronts walk through
-    const int per_cu = std::max(1, std::min(2, (int)(kMaxLds / lds)));
-    const int blocks = std::min((groups + kWaves - 1) / kWaves, ctx->compute_units * per_cu);
+    // one workgroup per compute unit at most: its staging serves all the rows its wavefronts walk through
+    const int groups = (w.rows + kR - 1) / kR, blocks = std::min((groups + kWaves - 1) / kWaves, ctx->compute_units);
     skn_launch(ctx, dense_matvec_kernel<W, MODE>, dim3((unsigned)blocks), dim3(kThreads), lds, (const W*)w.w, w.rows, w.k_pad, plane, w.bias, src, out);
     SKN_LAUNCH_CHECK(ctx);
     return SKN_OK;
@@ -281,12 +292,19 @@ int launch_mode(skn_ctx* ctx, const skn_dense_mat& w, const skn_matvec_src& src,
     return launch<W, SKN_XSRC_PLAIN>(ctx, w, src, out);
 }
 
-int dense_matvec_init(skn_ctx* ctx) {
-    const void* fns[] = {(const void*)dense_matvec_kernel<uint16_t, SKN_XSRC_PLAIN>, (const void*)dense_matvec_kernel<uint16_t, SKN_XSRC_GROUP_NORM>,
-                         (const void*)dense_matvec_kernel<uint16_t, SKN_XSRC_MERGE>, (const void*)dense_matvec_kernel<float, SKN_XSRC_PLAIN>,
-                         (const void*)dense_matvec_kernel<float, SKN_XSRC_GROUP_NORM>, (const void*)dense_matvec_kernel<float, SKN_XSRC_MERGE>};
-    for (const void* f : fns) SKN_HIP(ctx, hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, kMaxLds));
+template <typename W, int MODE>
+int allow_lds(skn_ctx* ctx) {
+    SKN_HIP(ctx, hipFuncSetAttribute((const void*)dense_matvec_kernel<W, MODE>, hipFuncAttributeMaxDynamicSharedMemorySize, kMaxLds));
     return SKN_OK;
+}
+
+int dense_matvec_init(skn_ctx* ctx) {
+    SKN_TRY((allow_lds<uint16_t, SKN_XSRC_PLAIN>(ctx)));
+    SKN_TRY((allow_lds<uint16_t, SKN_XSRC_GROUP_NORM>(ctx)));
+    SKN_TRY((allow_lds<uint16_t, SKN_XSRC_MERGE>(ctx)));
+    SKN_TRY((allow_lds<float, SKN_XSRC_PLAIN>(ctx)));
+    SKN_TRY((allow_lds<float, SKN_XSRC_GROUP_NORM>(ctx)));
+    return allow_lds<float, SKN_XSRC_MERGE>(ctx);
 }
 skn_family register_family(dense_matvec_init);
 
@@ -300,7 +318,7 @@ int skn_dense_matvec(skn_ctx* ctx, const skn_dense_mat& w, const skn_matvec_src&
                 "dense matvec: bad second input");
     SKN_REQUIRE(ctx, src.mode != SKN_XSRC_GROUP_NORM || (src.norm_w && src.groups > 0 && src.groups <= kMaxGroups && src.k0 % src.groups == 0),
                 SKN_ERR_SHAPE, "dense matvec: %d norm groups of %d columns (at most %d groups)", src.groups, src.k0, kMaxGroups);
-    SKN_REQUIRE(ctx, src.mode != SKN_XSRC_MERGE || (src.ml && src.splits > 0 && src.heads * src.splits <= kMaxMerge && src.k0 == src.heads * src.dim &&
+    SKN_REQUIRE(ctx, src.mode != SKN_XSRC_MERGE || (src.ml && src.splits > 0 && src.splits <= kMaxSplits && src.heads * src.splits <= kMaxMerge && src.k0 == src.heads * src.dim &&
                                                      src.dim_pad % 4 == 0),
                 SKN_ERR_SHAPE, "dense matvec: cannot merge %d heads x %d splits", src.heads, src.splits);
     SKN_REQUIRE(ctx, out.nseg >= 0 && out.nseg <= kDenseMaxSegs && (out.nseg > 0 || out.resid), SKN_ERR_ARG, "dense matvec: no output");

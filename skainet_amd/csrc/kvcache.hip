@@ -188,6 +188,7 @@ int skn_kv_create_shared(skn_ctx* ctx, int n_seq, int n_head, int dim, int elem_
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_create_shared: ctx is null");
     SKN_REQUIRE(ctx, dim > 0 && dim <= 256, SKN_ERR_SHAPE, "skn_kv_create_shared: heads of %d elements (1 to 256)", dim);
     SKN_REQUIRE(ctx, elem_type == SKN_TYPE_F16 || elem_type == SKN_TYPE_F32, SKN_ERR_TYPE, "skn_kv_create_shared: type %d (F16 or F32)", elem_type);
+    SKN_REQUIRE(ctx, max_tokens <= 1 << 22, SKN_ERR_SHAPE, "skn_kv_create_shared: %d tokens (at most %d)", max_tokens, 1 << 22);
     return kv_create(ctx, n_seq, n_head, dim <= 64 ? 64 : dim <= 128 ? 128 : 256, page_tokens, max_tokens, true, elem_type, dim, out);
 }
 
