@@ -1,16 +1,21 @@
 // The generalized delta rule and the state it runs on (rstate.h).
 //
-// Everything here is fp32.  Value channels of a head are independent columns of its state, so a group of L lanes owns a
-// column: eight key channels per lane, the column's two dot products (with k before, with r after the update) are sums over
-// the L lanes by DPP, and the state never leaves the registers between two tokens.  Because u = k / |k|, the removal term
-// is (a k / |k|^2) (k^T S): one vector b = a k / (sum k^2 + 1e-6) beside k serves it.
+// Everything here is fp32, the matrix instructions (v_mfma_f32_16x16x4_f32) included.  Value channels of a head are independent
+// columns of its state.  Because u = k / |k|, the removal term is (a k / |k|^2) (k^T S): one vector b = a k / (sum k^2 + 1e-6)
+// beside k serves it.
 //
-// Prompts take two launches.  delta_pack_kernel writes, per head and token, the five vectors k, w, b, r, v one after the
-// other, padded to the lanes' channels (and tokens that change nothing up to whole blocks); delta_scan_kernel -- one small
-// workgroup per head and run of columns -- has the next 20 KB block of that stream on its way into registers while it computes
-// the tokens of the current one out of LDS, each token's vectors read one token ahead.  (Copied straight into LDS instead,
-// the compiler puts a wait for the copy in front of the next LDS read.)  The tokens of a sequence are a chain; what is
-// parallel are the heads and the columns.
+// Prompts take two launches, and sixteen tokens (a chunk) are one step of the chain.  With W(s, t) the product of the decays of
+// tokens s .. t of the chunk, S the state before it and y_t = k_t^T S_{t-1} what k_t reads,
+//   (I + beta) Y = K0 S + alpha V,    K0_t = k_t W(0, t-1),   alpha_ts, beta_ts = k_t^T W(s+1, t-1) {k_s, b_s} for s < t
+//   O = R0 S + gamma V - delta Y,     R0_t = r_t W(0, t),     gamma_ts, delta_ts = r_t^T W(s+1, t) {k_s, b_s} for s <= t
+//   S' = W(0, 15) S + sum_s k_s W(s+1, 15) v_s - b_s W(s+1, 15) y_s
+// delta_chunk_kernel -- one wavefront per chunk and head, all chunks at once, since none of it depends on the state -- forms the
+// four triangles on the matrix cores, solves with I + beta, and leaves
+//   Y = K1 S + A1 V,  O = R1 S + G1 V     (K1 = (I + beta)^-1 K0, A1 = (I + beta)^-1 alpha, R1 = R0 - delta K1, G1 = gamma - delta A1)
+// as operands in the order in which the matrix instructions take them.  delta_scan_kernel then walks the chunks with one
+// wavefront per head and sixteen columns, its part of S in accumulator layout -- which is also the layout of a column operand,
+// so S and Y are multiplied as they stand -- and no LDS, no barrier: a chunk's operands are coalesced loads one chunk ahead.
+// (Decays enter the triangles as ratios of products over at most sixteen tokens: any decay from 0.01 to 1 is safe in fp32.)
 // A decode step is one launch, one workgroup per head: the decay's low-rank product, the step, the head's norm and the gate.
 #include "dense.h"
 #include "rstate.h"
@@ -50,113 +55,254 @@ __device__ __forceinline__ float delta_column(Vec8& s, const Vec8& k, const Vec8
     return dot_over_lanes<L>(r, s);
 }
 
-constexpr int kVecs = 5;  // k, w, b, r, v
+typedef float f32x4 __attribute__((ext_vector_type(4)));
 
-constexpr int kBlockFloats = kVecs * 1024;  // a block of the packed stream: 1024 / dim_pad tokens
-constexpr int kTrash = 64;                  // floats behind the stream that lanes without a column store to
+constexpr int kChunk = 16;
+constexpr int kTrash = 64;  // floats behind the operands that take the outputs of tokens past the end
 
-__host__ __device__ inline int block_tokens(int dim_pad) { return 1024 / dim_pad; }
-__host__ __device__ inline int padded_tokens(int n, int dim_pad) { return (n + block_tokens(dim_pad) - 1) / block_tokens(dim_pad) * block_tokens(dim_pad); }
+// Operands of a chunk and head, in floats from its start.  Row operands (K1, R1: [token][channel], in tiles of 16 channels;
+// A1, G1: [token][token]): lane 16 q + t holds elements 4 q .. 4 q + 3 of row t.  kT, bT ([channel][token], b negated) and V
+// ([token][column] as a column operand): lane 16 q + c holds tokens 4 q .. 4 q + 3 of channel (column) c of the tile.
+__host__ __device__ constexpr int off_k1(int) { return 0; }
+__host__ __device__ constexpr int off_r1(int dp) { return 16 * dp; }
+__host__ __device__ constexpr int off_kt(int dp) { return 32 * dp; }
+__host__ __device__ constexpr int off_bt(int dp) { return 48 * dp; }
+__host__ __device__ constexpr int off_v(int dp) { return 64 * dp; }
+__host__ __device__ constexpr int off_a1(int dp) { return 80 * dp; }
+__host__ __device__ constexpr int off_g1(int dp) { return 80 * dp + 256; }
+__host__ __device__ constexpr int off_w(int dp) { return 80 * dp + 512; }
+__host__ __device__ constexpr int chunk_floats(int dp) { return 81 * dp + 512; }
 
-// one wavefront per (token, head); n_pad: tokens with those that only fill the last block (k = b = 0, w = 1)
-__global__ __launch_bounds__(256) void delta_pack_kernel(const float* __restrict__ r, const float* __restrict__ k, const float* __restrict__ v,
-                                                         const float* __restrict__ w, const float* __restrict__ a, int ld, int n, int n_pad, int heads,
-                                                         int dim, int dim_pad, float* __restrict__ pack) {
-    const int id = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    if (id >= n_pad * heads) return;
-    const int t = id / heads, h = id - t * heads;
-    const int64_t at = (int64_t)min(t, n - 1) * ld + h * dim;
-    float kk[4], ss = 0.f;
+__device__ __forceinline__ f32x4 mma(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+__device__ __forceinline__ f32x4 load4(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
+
+// N sums over the wavefront, step by step for all of them
+template <int N>
+__device__ __forceinline__ void wave_sums(float (&x)[N]) {
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-        const int d = lane + 64 * i;
-        kk[i] = d < dim ? k[at + d] : 0.f;
-        ss = fmaf(kk[i], kk[i], ss);
+    for (int i = 0; i < N; i++) x[i] = lane_group_sum<16>(x[i]);
+#pragma unroll
+    for (int i = 0; i < N; i++) {
+        const auto r = __builtin_amdgcn_permlane16_swap(__float_as_uint(x[i]), __float_as_uint(x[i]), false, false);
+        x[i] = __uint_as_float(r[0]) + __uint_as_float(r[1]);
     }
-    const float inv = 1.0f / (wave_sum(ss) + kUnitEps);
-    float* out = pack + ((int64_t)h * n_pad + t) * kVecs * dim_pad;
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-        const int d = lane + 64 * i;
-        if (d >= dim_pad) continue;
-        const bool in = d < dim && t < n;
-        out[d] = in ? kk[i] : 0.f;
-        out[dim_pad + d] = in ? w[at + d] : 1.f;
-        out[2 * dim_pad + d] = in ? a[at + d] * kk[i] * inv : 0.f;
-        out[3 * dim_pad + d] = in ? r[at + d] : 0.f;
-        out[4 * dim_pad + d] = in ? v[at + d] : 0.f;
+    for (int i = 0; i < N; i++) {
+        const auto r = __builtin_amdgcn_permlane32_swap(__float_as_uint(x[i]), __float_as_uint(x[i]), false, false);
+        x[i] = __uint_as_float(r[0]) + __uint_as_float(r[1]);
     }
 }
 
-// grid (column runs, heads); NW wavefronts of 64 / L columns each
-template <int L, int NW>
-__global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __restrict__ pack, int n, int n_pad, int heads, int dim,
-                                                             float* __restrict__ state, float* __restrict__ o, float* __restrict__ trash) {
-    __shared__ __align__(16) float lds[2][kBlockFloats];
-    constexpr int DP = 8 * L, C = 1024 / DP, kTurns = kBlockFloats / 4 / (64 * NW);  // float4 per thread and block
-    static_assert(kTurns * 4 * 64 * NW == kBlockFloats, "a block is whole float4 per thread");
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.y;
-    const int rl = lane & (L - 1);
-    const int col = (blockIdx.x * NW + wave) * (64 / L) + lane / L;
-    const bool live = col < dim;
-    const int colc = min(col, dim - 1);
-    float* sp = state + ((int64_t)h * dim + colc) * DP + 8 * rl;
-    Vec8 s;
-    s.load(sp);
-    const float4* src = reinterpret_cast<const float4*>(pack + (int64_t)h * n_pad * kVecs * DP) + tid;
-    const int blocks = n_pad / C;
-    float4 ahead[kTurns];
+// x_t = rhs_t - sum_{s < t} beta_ts x_s, then z_t - sum_{s <= t} delta_ts x_s, for this lane's column; rows of rhs and z at
+// pitch, replaced by the results
+__device__ __forceinline__ void solve_column(float* rhs, float* z, int pitch, const float (*beta)[20], const float (*delta)[20]) {
+    float x[kChunk];
 #pragma unroll
-    for (int i = 0; i < kTurns; i++) ahead[i] = src[i * 64 * NW];
+    for (int t = 0; t < kChunk; t++) {
+        x[t] = rhs[t * pitch];
+#pragma unroll
+        for (int s = 0; s < t; s++) x[t] = fmaf(-beta[t][s], x[s], x[t]);
+        rhs[t * pitch] = x[t];
+    }
+#pragma unroll
+    for (int t = 0; t < kChunk; t++) {
+        float o = z[t * pitch];
+#pragma unroll
+        for (int s = 0; s <= t; s++) o = fmaf(-delta[t][s], x[s], o);
+        z[t * pitch] = o;
+    }
+}
 
-    struct Token {
-        Vec8 k, w, b, r;
-        float v;
-    };
-    for (int blk = 0; blk < blocks; blk++) {
-        // (this buffer was last read two blocks ago, and everyone has passed the barrier since)
-        float4* dst = reinterpret_cast<float4*>(lds[blk & 1]) + tid;
+// one wavefront per (chunk, head); tokens past n change nothing (k = b = r = v = 0, decay 1)
+template <int DP>
+__global__ __launch_bounds__(64) void delta_chunk_kernel(const float* __restrict__ r, const float* __restrict__ k, const float* __restrict__ v,
+                                                         const float* __restrict__ w, const float* __restrict__ a, int ld, int n, int heads, int dim,
+                                                         float* __restrict__ ops) {
+    constexpr int kPitch = DP + 4, kSets = (DP + 63) / 64, kTiles = DP / 16;
+    __shared__ __align__(16) float row[4][kChunk * kPitch];  // K0 then K1, R0 then R1, k / W, b / W
+    __shared__ __align__(16) float tri[4][kChunk][20];       // alpha then A1, gamma then G1, beta, delta
+    const int lane = threadIdx.x, chunk = blockIdx.x, h = blockIdx.y, chunks = gridDim.x, t0 = chunk * kChunk;
+    float* out = ops + ((int64_t)h * chunks + chunk) * chunk_floats(DP);
+    float inv[kChunk];
 #pragma unroll
-        for (int i = 0; i < kTurns; i++) dst[i * 64 * NW] = ahead[i];
-        const float4* next = src + (int64_t)min(blk + 1, blocks - 1) * (kBlockFloats / 4);
+    for (int t = 0; t < kChunk; t++) {
+        inv[t] = 0.f;
+        const float* kr = k + (int64_t)min(t0 + t, n - 1) * ld + h * dim;
 #pragma unroll
-        for (int i = 0; i < kTurns; i++) ahead[i] = next[i * 64 * NW];
-        __builtin_amdgcn_sched_barrier(0);
-        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-        const float* base = lds[blk & 1];
-        const int t0 = blk * C;
-        auto read = [&](Token& x, int t) __attribute__((always_inline)) {
-            const float* p = base + t * kVecs * DP;
-            x.k.load(p + 8 * rl);
-            x.w.load(p + DP + 8 * rl);
-            x.b.load(p + 2 * DP + 8 * rl);
-            x.r.load(p + 3 * DP + 8 * rl);
-            x.v = p[4 * DP + colc];
-        };
-        Token even, odd;
-        read(even, 0);
-        constexpr int G = L < C ? L : C;  // the L lanes of a column keep the outputs of G tokens and store them together
-        float keep = 0.f;
-#pragma unroll
-        for (int t = 0; t < C; t += 2) {
-            read(odd, t + 1);
-            __builtin_amdgcn_sched_barrier(0);
-            const float o0 = delta_column<L>(s, even.k, even.w, even.b, even.r, even.v);
-            keep = rl == t % G ? o0 : keep;
-            if (t + 2 < C) read(even, t + 2);
-            __builtin_amdgcn_sched_barrier(0);
-            const float o1 = delta_column<L>(s, odd.k, odd.w, odd.b, odd.r, odd.v);
-            keep = rl == t % G + 1 ? o1 : keep;
-            if ((t + 2) % G == 0) {
-                // (one store whatever the lane: a skipped one would leave the number of requests outstanding unknown, and
-                // the wait for the next block would wait for every store)
-                const int mine = t0 + t + 2 - G + rl;
-                float* p = live && rl < G && mine < n ? o + ((int64_t)mine * heads + h) * dim + col : trash + lane;
-                *p = keep;
-            }
+        for (int i = 0; i < kSets; i++) {
+            const float x = lane + 64 * i < dim ? kr[lane + 64 * i] : 0.f;
+            inv[t] = fmaf(x, x, inv[t]);
         }
     }
-    if (live) s.store(sp);
+    wave_sums<kChunk>(inv);
+#pragma unroll
+    for (int t = 0; t < kChunk; t++) inv[t] = 1.0f / (inv[t] + kUnitEps);
+
+#pragma unroll 1
+    for (int i = 0; i < kSets; i++) {
+        const int d = lane + 64 * i;
+        if (d >= DP) continue;
+        float kk[kChunk], bb[kChunk], vv[kChunk], upto = 1.f;  // upto: W(0, t)
+#pragma unroll
+        for (int t = 0; t < kChunk; t++) {
+            const bool in = d < dim && t0 + t < n;
+            const int64_t at = (int64_t)min(t0 + t, n - 1) * ld + h * dim + min(d, dim - 1);
+            const float kt = in ? k[at] : 0.f, wt = in ? w[at] : 1.f, bt = in ? a[at] * kt * inv[t] : 0.f, rt = in ? r[at] : 0.f;
+            vv[t] = in ? v[at] : 0.f;
+            row[0][t * kPitch + d] = kt * upto;
+            upto *= wt;
+            row[1][t * kPitch + d] = rt * upto;
+            const float rec = 1.0f / upto;
+            kk[t] = kt * rec;
+            bb[t] = bt * rec;
+            row[2][t * kPitch + d] = kk[t];
+            row[3][t * kPitch + d] = bb[t];
+        }
+        out[off_w(DP) + d] = upto;
+        // tile d / 16, lane 16 q + d % 16
+        float* frag = out + ((d >> 4) * 64 + (d & 15)) * 4;
+#pragma unroll
+        for (int q = 0; q < 4; q++) {
+            const f32x4 x = {kk[4 * q] * upto, kk[4 * q + 1] * upto, kk[4 * q + 2] * upto, kk[4 * q + 3] * upto};
+            const f32x4 y = {-bb[4 * q] * upto, -bb[4 * q + 1] * upto, -bb[4 * q + 2] * upto, -bb[4 * q + 3] * upto};
+            const f32x4 z = {vv[4 * q], vv[4 * q + 1], vv[4 * q + 2], vv[4 * q + 3]};
+            *reinterpret_cast<f32x4*>(frag + off_kt(DP) + 64 * q) = x;
+            *reinterpret_cast<f32x4*>(frag + off_bt(DP) + 64 * q) = y;
+            *reinterpret_cast<f32x4*>(frag + off_v(DP) + 64 * q) = z;
+        }
+    }
+    __syncthreads();
+    // the triangles: rows K0, R0 times columns k / W, b / W
+    const int t16 = lane & 15, q4 = lane >> 4;
+    f32x4 g[4];  // alpha, gamma, beta, delta
+#pragma unroll
+    for (int i = 0; i < 4; i++) g[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+    for (int c = 0; c < kTiles; c++) {
+        const int at = t16 * kPitch + 16 * c + 4 * q4;
+        const f32x4 k0 = load4(&row[0][at]), r0 = load4(&row[1][at]), kw = load4(&row[2][at]), bw = load4(&row[3][at]);
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            g[0] = mma(k0[e], kw[e], g[0]);
+            g[1] = mma(r0[e], kw[e], g[1]);
+            g[2] = mma(k0[e], bw[e], g[2]);
+            g[3] = mma(r0[e], bw[e], g[3]);
+        }
+    }
+#pragma unroll
+    for (int e = 0; e < 4; e++) {
+        const int t = 4 * q4 + e, s = t16;
+        tri[0][t][s] = s < t ? g[0][e] : 0.f;
+        tri[1][t][s] = s <= t ? g[1][e] : 0.f;
+        tri[2][t][s] = s < t ? g[2][e] : 0.f;
+        tri[3][t][s] = s <= t ? g[3][e] : 0.f;
+    }
+    __syncthreads();
+#pragma unroll 1
+    for (int i = 0; i < kSets; i++) {
+        const int d = lane + 64 * i;
+        if (d < DP) solve_column(&row[0][d], &row[1][d], kPitch, tri[2], tri[3]);
+    }
+    if (lane < kChunk) solve_column(&tri[0][0][lane], &tri[1][0][lane], 20, tri[2], tri[3]);
+    __syncthreads();
+#pragma unroll 2
+    for (int c = 0; c < kTiles; c++) {
+        *reinterpret_cast<f32x4*>(out + off_k1(DP) + (c * 64 + lane) * 4) = load4(&row[0][t16 * kPitch + 16 * c + 4 * q4]);
+        *reinterpret_cast<f32x4*>(out + off_r1(DP) + (c * 64 + lane) * 4) = load4(&row[1][t16 * kPitch + 16 * c + 4 * q4]);
+    }
+    *reinterpret_cast<f32x4*>(out + off_a1(DP) + lane * 4) = load4(&tri[0][t16][4 * q4]);
+    *reinterpret_cast<f32x4*>(out + off_g1(DP) + lane * 4) = load4(&tri[1][t16][4 * q4]);
+}
+
+template <int DP>
+struct ChunkOps {
+    static constexpr int kTiles = DP / 16;
+    f32x4 k1[kTiles], r1[kTiles], kt[kTiles], bt[kTiles], w[kTiles], v, a1, g1;
+    __device__ __forceinline__ void load(const float* p, int lane, int tile) {
+#pragma unroll
+        for (int j = 0; j < kTiles; j++) {
+            k1[j] = load4(p + off_k1(DP) + (j * 64 + lane) * 4);
+            r1[j] = load4(p + off_r1(DP) + (j * 64 + lane) * 4);
+        }
+        v = load4(p + off_v(DP) + (tile * 64 + lane) * 4);
+        a1 = load4(p + off_a1(DP) + lane * 4);
+        g1 = load4(p + off_g1(DP) + lane * 4);
+#pragma unroll
+        for (int j = 0; j < kTiles; j++) {
+            kt[j] = load4(p + off_kt(DP) + (j * 64 + lane) * 4);
+            bt[j] = load4(p + off_bt(DP) + (j * 64 + lane) * 4);
+            w[j] = load4(p + off_w(DP) + 16 * j + 4 * (lane >> 4));
+        }
+    }
+};
+
+// One wavefront per head and tile of sixteen columns.  The wavefronts of a head are on one XCD (blockIdx % 8): they read the
+// same operands, which then come from memory once.
+template <int DP>
+__global__ __launch_bounds__(64) void delta_scan_kernel(const float* __restrict__ ops, int n, int chunks, int heads, int dim, float* __restrict__ state,
+                                                        float* __restrict__ o, float* __restrict__ trash) {
+    constexpr int kTiles = DP / 16;
+    const int lane = threadIdx.x, tiles = (dim + 15) / 16, turn = (int)(blockIdx.x >> 3), h = (int)(blockIdx.x & 7) + 8 * (turn / tiles), tile = turn % tiles;
+    if (h >= heads) return;
+    // (lanes beyond the last column compute along on zeros of V and store nothing)
+    const int col = 16 * tile + (lane & 15);
+    const bool live = col < dim;
+    float* sp = state + ((int64_t)h * dim + min(col, dim - 1)) * DP + 4 * (lane >> 4);
+    f32x4 s[kTiles];
+#pragma unroll
+    for (int j = 0; j < kTiles; j++) s[j] = load4(sp + 16 * j);
+    const float* src = ops + (int64_t)h * chunks * chunk_floats(DP);
+
+    auto step = [&](const ChunkOps<DP>& x, int chunk) __attribute__((always_inline)) {
+        f32x4 y = {0.f, 0.f, 0.f, 0.f}, z = y;
+#pragma unroll
+        for (int e = 0; e < 4; e++) y = mma(x.a1[e], x.v[e], y), z = mma(x.g1[e], x.v[e], z);
+#pragma unroll
+        for (int j = 0; j < kTiles; j++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) y = mma(x.k1[j][e], s[j][e], y), z = mma(x.r1[j][e], s[j][e], z);
+#pragma unroll
+        for (int j = 0; j < kTiles; j++) s[j] *= x.w[j];
+#pragma unroll
+        for (int e = 0; e < 4; e++)
+#pragma unroll
+            for (int j = 0; j < kTiles; j++) s[j] = mma(x.kt[j][e], x.v[e], s[j]);
+#pragma unroll
+        for (int e = 0; e < 4; e++)
+#pragma unroll
+            for (int j = 0; j < kTiles; j++) s[j] = mma(x.bt[j][e], y[e], s[j]);
+        // (one store per token whatever the lane: a skipped one would leave the number of requests outstanding unknown, and
+        // the wait for the next chunk's operands would wait for the stores)
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int t = chunk * kChunk + 4 * (lane >> 4) + e;
+            float* dst = live && t < n ? o + ((int64_t)t * heads + h) * dim + col : trash + lane;
+            *dst = z[e];
+        }
+    };
+    ChunkOps<DP> even;
+    if constexpr (DP <= 128) {
+        ChunkOps<DP> odd;
+        even.load(src, lane, tile);
+        for (int c = 0; c < chunks; c += 2) {
+            odd.load(src + (int64_t)min(c + 1, chunks - 1) * chunk_floats(DP), lane, tile);
+            __builtin_amdgcn_sched_barrier(0);
+            step(even, c);
+            if (c + 1 == chunks) break;
+            even.load(src + (int64_t)min(c + 2, chunks - 1) * chunk_floats(DP), lane, tile);
+            __builtin_amdgcn_sched_barrier(0);
+            step(odd, c + 1);
+        }
+    } else {
+        for (int c = 0; c < chunks; c++) {
+            even.load(src + (int64_t)c * chunk_floats(DP), lane, tile);
+            step(even, c);
+        }
+    }
+    if (live) {
+#pragma unroll
+        for (int j = 0; j < kTiles; j++) *reinterpret_cast<f32x4*>(sp + 16 * j) = s[j];
+    }
 }
 
 // one wavefront per (token, head)
@@ -190,7 +336,7 @@ template <int L, int NW, typename W>
 __global__ __launch_bounds__(64 * NW) void delta_step_kernel(const skn_delta_step p, int dim, float* __restrict__ state) {
     constexpr int DP = 8 * L, CW = 64 / L, kThreads = 64 * NW;  // columns per wavefront
     constexpr int kPasses = (DP + NW * CW - 1) / (NW * CW);
-    __shared__ __align__(16) float vec[kVecs][DP];
+    __shared__ __align__(16) float vec[5][DP];  // k, w, b, r, v
     __shared__ float so[DP], red[NW];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x, rl = lane & (L - 1);
     const int off = h * dim;
@@ -263,12 +409,15 @@ __global__ __launch_bounds__(64 * NW) void delta_step_kernel(const skn_delta_ste
     for (int d = tid; d < dim; d += kThreads) p.y[off + d] = so[d] * inv * p.norm[off + d] * p.g[off + d];
 }
 
-template <int L, int NW>
-int launch_scan(skn_ctx* ctx, const skn_rstate* st, const float* pack, int n, float* state, float* o) {
-    const int per_wg = NW * (64 / L), n_pad = padded_tokens(n, st->dim_pad);
-    float* trash = const_cast<float*>(pack) + (size_t)n_pad * st->heads * kVecs * st->dim_pad;
-    skn_launch(ctx, delta_scan_kernel<L, NW>, dim3((st->dim + per_wg - 1) / per_wg, st->heads), dim3(64 * NW), 0, pack, n, n_pad, st->heads, st->dim, state,
-               o, trash);
+template <int DP>
+int launch_rows(skn_ctx* ctx, const skn_rstate* st, const float* r, const float* k, const float* v, const float* w, const float* a, int ld, int n, float* ops,
+                float* state, float* o) {
+    const int chunks = (n + kChunk - 1) / kChunk, tiles = (st->dim + 15) / 16;
+    skn_launch(ctx, delta_chunk_kernel<DP>, dim3(chunks, st->heads), dim3(64), 0, r, k, v, w, a, ld, n, st->heads, st->dim, ops);
+    SKN_LAUNCH_CHECK(ctx);
+    float* trash = ops + (size_t)chunks * st->heads * chunk_floats(DP);
+    skn_launch(ctx, delta_scan_kernel<DP>, dim3((unsigned)((st->heads + 7) / 8 * 8 * tiles)), dim3(64), 0, (const float*)ops, n, chunks, st->heads, st->dim, state, o,
+               trash);
     SKN_LAUNCH_CHECK(ctx);
     return SKN_OK;
 }
@@ -281,16 +430,6 @@ int launch_step(skn_ctx* ctx, const skn_rstate* st, const skn_delta_step& p, flo
     return SKN_OK;
 }
 
-template <int L>
-int scan_waves(skn_ctx* ctx, const skn_rstate* st, const float* pack, int n, float* state, float* o) {
-    // one wavefront per workgroup spreads the columns over the compute units; four share the copied stream when there
-    // are more column runs than compute units
-    const int runs = st->heads * ((st->dim * L + 63) / 64);
-    if (runs > 2 * ctx->compute_units) return launch_scan<L, 4>(ctx, st, pack, n, state, o);
-    if (runs > ctx->compute_units) return launch_scan<L, 2>(ctx, st, pack, n, state, o);
-    return launch_scan<L, 1>(ctx, st, pack, n, state, o);
-}
-
 __global__ void fill_zero_kernel(float4* p, int64_t n) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i < n) p[i] = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -299,22 +438,18 @@ __global__ void fill_zero_kernel(float4* p, int64_t n) {
 }  // namespace
 
 size_t skn_delta_pack_floats(const skn_rstate* st, int n) {
-    return (size_t)padded_tokens(n, st->dim_pad) * st->heads * kVecs * st->dim_pad + kTrash;
+    return (size_t)((n + kChunk - 1) / kChunk) * st->heads * chunk_floats(st->dim_pad) + kTrash;
 }
 
 int skn_delta_rows(skn_ctx* ctx, skn_rstate* st, int seq, const float* r, const float* k, const float* v, const float* w, const float* a, int ld, int n,
                    float* pack, float* o) {
-    SKN_REQUIRE(ctx, n > 0 && (int64_t)(n + 32) * st->heads < ((int64_t)1 << 31) - 4, SKN_ERR_SHAPE, "delta rule: %d tokens x %d heads", n, st->heads);
-    const int n_pad = padded_tokens(n, st->dim_pad);
-    skn_launch(ctx, delta_pack_kernel, dim3((unsigned)(((int64_t)n_pad * st->heads + 3) / 4)), dim3(256), 0, r, k, v, w, a, ld, n, n_pad, st->heads, st->dim,
-               st->dim_pad, pack);
-    SKN_LAUNCH_CHECK(ctx);
+    SKN_REQUIRE(ctx, n > 0 && st->heads <= 65535, SKN_ERR_SHAPE, "delta rule: %d tokens x %d heads", n, st->heads);
     float* s = st->seq_state(seq);
     switch (st->dim_pad) {
-        case 32: return scan_waves<4>(ctx, st, pack, n, s, o);
-        case 64: return scan_waves<8>(ctx, st, pack, n, s, o);
-        case 128: return scan_waves<16>(ctx, st, pack, n, s, o);
-        default: return scan_waves<32>(ctx, st, pack, n, s, o);
+        case 32: return launch_rows<32>(ctx, st, r, k, v, w, a, ld, n, pack, s, o);
+        case 64: return launch_rows<64>(ctx, st, r, k, v, w, a, ld, n, pack, s, o);
+        case 128: return launch_rows<128>(ctx, st, r, k, v, w, a, ld, n, pack, s, o);
+        default: return launch_rows<256>(ctx, st, r, k, v, w, a, ld, n, pack, s, o);
     }
 }
 
