@@ -85,12 +85,12 @@ def check(got, want, dtype, what=None):
     assert over <= (len(err) // 50 if dtype == "bfloat16" else 0) and err.max() < 3 * tol, (what, over, int(err.argmax()), err.max())
 
 
-def finder(heads, kv_heads, dim, seed=0):
+def finder(heads, kv_heads, dim, seed=0, match=14.0):
     """One attention layer in which the last token's query (ASK) finds the key of one other token (RARE), whose value is unlike
     any other: keys read the first half of the normalised stream, queries the second half through the same matrices, and
     ASK's second half is RARE's first.  The scale lets a match outweigh hundreds of other keys and, in the heads with flat
     slopes, its distance."""
-    cfg = model([attention(heads, kv_heads, dim, scale=14.0 / dim, q_temp=(0.05, 64), ff=0)], width=96, vocab=61, groups=2, mult=1.0)
+    cfg = model([attention(heads, kv_heads, dim, scale=match / dim, q_temp=(0.05, 64), ff=0)], width=96, vocab=61, groups=2, mult=1.0)
     w = weights(cfg, 1, seed)
     k = w["l0.mix.k"].reshape(kv_heads, dim, 96) * 2 ** 0.5
     k[:, :, 48:] = 0

@@ -96,6 +96,26 @@ def test_a_far_key_is_found_in_prompts_and_in_decoding(hip, heads, kv_heads, dim
     m.free()
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("heads,kv_heads,dim", [(6, 2, 48), (5, 5, 9), (4, 1, 100), (2, 2, 200), (24, 2, 64)])
+def test_decoding_over_contexts_that_are_split(hip, heads, kv_heads, dim, dtype):
+    """Contexts past 512 and 1024 tokens: several workgroups share a head's keys and the output product's staging merges them."""
+    cfg, w = cases.finder(heads, kv_heads, dim, match=22.0)
+    n = 1100
+    toks = [t % cases.COMMON for t in cases.tokens(cfg, n, seed=7)]
+    m = cases.device_model(hip, cfg, w, dtype, max_tokens=1200, page_tokens=64)
+    for far in (0, 63, 64, 511, 512, 1023, 1024):
+        t = list(toks)
+        t[far], t[-1] = cases.RARE, cases.ASK
+        want = orc.forward(cfg, w, t)
+        other = list(t)
+        other[far] = cases.COMMON
+        assert cases.logit_error(orc.forward(cfg, w, other)[-1:], want[-1:])[0] > 5 * cases.TOLERANCE[dtype]
+        got = run(m, t, [n - 12] + [1] * 12, want=range(n - 14, n))
+        cases.check(got, want[n - 14:], dtype, far)
+    m.free()
+
+
 def test_requests_one_after_the_other_use_pages_and_states_again(hip):
     cfg, rank = cases.MODELS["mixed"]
     w = cases.weights(cfg, rank)

@@ -15,7 +15,7 @@ def rel(got, want):
 
 # ---- norm and activation -----------------------------------------------------------------------------------------------
 
-@pytest.mark.parametrize("rows,n,groups", [(1, 64, 1), (3, 45, 9), (5, 192, 2), (2, 4096, 4), (4, 1000, 8), (7, 30, 30), (2, 257, 1)])
+@pytest.mark.parametrize("rows,n,groups", [(1, 64, 1), (3, 45, 9), (5, 200, 2), (2, 4096, 4), (4, 1000, 8), (7, 30, 30), (2, 257, 1)])
 def test_grouped_norm(hip, rows, n, groups):
     rng = np.random.default_rng(n + groups)
     x = (rng.standard_normal((rows, n)) * np.exp(rng.standard_normal((rows, 1)))).astype(np.float32)
@@ -95,11 +95,11 @@ def test_shared_attention_in_one_go_in_portions_and_token_by_token(hip, heads, k
 @pytest.mark.parametrize("far", [0, 1, 15, 16, 17, 31, 32, 63, 64, 127, 128, 254, 255, 256])
 def test_one_far_key_stands_out(hip, elem, far):
     """Query 299 matches one key far away so well that it outweighs its distance: at page borders, tile borders, the first tokens."""
-    heads, kv_heads, dim, n = 4, 2, 64, 300
+    heads, kv_heads, dim, n = 6, 2, 56, 300
     q, k, p = attn_case(heads, kv_heads, dim, n, seed=5, coef=0.0, scale=1.0)
     p["q_norm"][:], p["k_norm"][:] = 1.0, 1.0
     qh = q[299].reshape(heads, dim)
-    k[far] = np.concatenate([qh[1], qh[3]])  # (head 1 reads cached head 0, head 3 cached head 1)
+    k[far] = np.concatenate([qh[2], qh[5]])  # (head 2 reads cached head 0, head 5 cached head 1)
     want = attn_oracle(q, k, p, heads, kv_heads, dim)
     without = k.copy()
     without[far] = -k[far]
@@ -217,8 +217,8 @@ def test_states_of_several_sequences_stay_apart_and_reset(hip):
     st.free()
 
 
-def test_many_heads_take_the_shared_workgroups(hip):
-    heads, dim, n = 80, 64, 33  # (more column runs than compute units)
+def test_many_heads(hip):
+    heads, dim, n = 80, 64, 33
     c = delta_case(heads, dim, n, seed=9)
     st = runtime.RecurrentState(hip, 1, heads, dim)
     assert rel(st.advance(0, *c), delta_oracle(c, heads, dim)) < 1e-5
