@@ -14,7 +14,7 @@ import java.lang.foreign.ValueLayout.JAVA_LONG
 import java.lang.invoke.MethodHandle
 
 object SknLib {
-    const val ABI_VERSION = 4
+    const val ABI_VERSION = 5
     const val OK = 0
     const val ERR_ARG = -1
     const val ERR_TYPE = -2
@@ -90,8 +90,15 @@ object SknLib {
     val rstateFree: MethodHandle = h("skn_rstate_free", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS))
     val rstateReset: MethodHandle = h("skn_rstate_reset", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_INT))
     val deltaRule: MethodHandle = h("skn_delta_rule", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_INT, ADDRESS, ADDRESS, ADDRESS, ADDRESS, ADDRESS, JAVA_INT, ADDRESS))
+    val kvCreateRanged: MethodHandle = h("skn_kv_create_ranged", FunctionDescriptor.of(JAVA_INT, ADDRESS, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, ADDRESS))
+    val attnRanged: MethodHandle = h("skn_attn_ranged", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_INT, ADDRESS, ADDRESS, ADDRESS, ADDRESS, ADDRESS, JAVA_INT, ADDRESS))
+    val kvCreateLatent: MethodHandle = h("skn_kv_create_latent", FunctionDescriptor.of(JAVA_INT, ADDRESS, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, ADDRESS))
+    val attnLatent: MethodHandle = h("skn_attn_latent", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_INT, ADDRESS, ADDRESS, ADDRESS, JAVA_INT, ADDRESS))
+    val rstateCreateConv: MethodHandle = h("skn_rstate_create_conv", FunctionDescriptor.of(JAVA_INT, ADDRESS, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_INT, ADDRESS))
+    val gatedDelta: MethodHandle = h("skn_gated_delta", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_INT, ADDRESS, ADDRESS, ADDRESS, ADDRESS, ADDRESS, ADDRESS, JAVA_INT, ADDRESS))
     val rmsnormGrouped: MethodHandle = h("skn_rmsnorm_grouped", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, ADDRESS, JAVA_INT, JAVA_INT, JAVA_INT, JAVA_FLOAT, ADDRESS))
     val xielu: MethodHandle = h("skn_xielu", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_LONG, JAVA_FLOAT, JAVA_FLOAT, ADDRESS))
+    val gelu: MethodHandle = h("skn_gelu", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, JAVA_LONG, ADDRESS))
     val hybridCreate: MethodHandle = h("skn_hybrid_create", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS, ADDRESS, ADDRESS))
     val hybridFree: MethodHandle = h("skn_hybrid_free", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS))
     val hybridReset: MethodHandle = h("skn_hybrid_reset", FunctionDescriptor.of(JAVA_INT, ADDRESS, ADDRESS))

@@ -22,7 +22,8 @@ LIB = os.path.join(HERE, "libskainet_hip.so")
 DENSE_LIB = os.path.join(HERE, "libskainet_dense.so")
 # the sources of the layer-list decoder over bf16 / fp32 weights and of nothing else (seconds to compile; the
 # block-quantized matvecs alone take minutes)
-DENSE_SOURCES = ("api", "kvcache", "stepper", "dense_gemm", "dense_matvec", "dense_rows", "attention_prefill", "attention_shared", "delta", "hybrid")
+DENSE_SOURCES = ("api", "kvcache", "stepper", "dense_gemm", "dense_matvec", "dense_rows", "attention_prefill", "attention_shared",
+                 "attention_ranged", "attention_latent", "delta", "gated_delta", "hybrid")
 
 ARCH = "gfx950"
 # packed-fp32 VALU forms are kept off: scalar fp32 code must not be fused into v_pk_* instructions

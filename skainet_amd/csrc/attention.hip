@@ -373,7 +373,7 @@ int skn_attn_launch_ex(skn_ctx* ctx, skn_kv* kv, const float* q_dev, const int32
                        int seq_fixed, int n_splits, float* partial, int* counters, float scale, float* out_dev,
                        int n_q_head) {
     const int D = kv->head_dim;
-    SKN_REQUIRE(ctx, !kv->shared, SKN_ERR_STATE, "attention: the cache shares its keys and values (skn_attn_shared reads it)");
+    SKN_REQUIRE(ctx, kv->kind == SKN_KV_PLAIN, SKN_ERR_STATE, "attention: not a cache of fp16 keys and values (skn_attn_shared, _ranged and _latent read the others)");
     if (n_q_head <= 0) n_q_head = kv->n_head;
     SKN_REQUIRE(ctx, n_q_head % kv->n_head == 0, SKN_ERR_SHAPE,
                 "attention: %d query heads are not a multiple of the %d cached heads", n_q_head, kv->n_head);
@@ -408,7 +408,7 @@ int skn_attn_launch_ex(skn_ctx* ctx, skn_kv* kv, const float* q_dev, const int32
 int skn_attn_launch_unmerged(skn_ctx* ctx, skn_kv* kv, const float* q_dev, const int32_t* nctx_dev, int n_queries,
                              int seq_fixed, int n_splits, float* opart, float* ml, float scale, float* out_dev, int n_q_head) {
     const int D = kv->head_dim;
-    SKN_REQUIRE(ctx, !kv->shared, SKN_ERR_STATE, "attention: the cache shares its keys and values (skn_attn_shared reads it)");
+    SKN_REQUIRE(ctx, kv->kind == SKN_KV_PLAIN, SKN_ERR_STATE, "attention: not a cache of fp16 keys and values (skn_attn_shared, _ranged and _latent read the others)");
     if (n_q_head <= 0) n_q_head = kv->n_head;
     SKN_REQUIRE(ctx, n_q_head % kv->n_head == 0, SKN_ERR_SHAPE,
                 "attention: %d query heads are not a multiple of the %d cached heads", n_q_head, kv->n_head);

@@ -11,6 +11,7 @@
 // Token streams as in csrc/attention.hip: a row is spread over head_dim / 8 lanes, the lanes of a row own a private softmax
 // stream per query head, nothing is staged and no barrier is met while tokens stream.  A step's launch computes the two
 // norms of its own token in its prologue (every workgroup for itself, from L2) while its first rows are on their way.
+#include "attention_stream.h"
 #include "dense.h"
 #include "kv.h"
 
@@ -18,42 +19,9 @@
 
 namespace {
 
-typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
-typedef _Float16 half2_t __attribute__((ext_vector_type(2)));
-
 constexpr int kThreads = 1024, kWaves = kThreads / 64;
 constexpr int kU = 4;           // rows per stream in flight
 constexpr int kMaxSplits = 16;  // what the merge in the output projection's staging is fed at most
-constexpr float kLog2e = 1.4426950408889634f;
-
-template <typename E>
-struct Row8;  // eight elements of a cached row
-template <>
-struct Row8<uint16_t> {
-    u32x4 a;
-    __device__ __forceinline__ void load(const uint16_t* p) { a = *reinterpret_cast<const u32x4*>(p); }
-    __device__ __forceinline__ void get(float (&f)[8]) const {
-#pragma unroll
-        for (int j = 0; j < 4; j++) {
-            const uint32_t w = a[j];  // (a bit cast applied directly to a vector element reads element 0)
-            const half2_t h = __builtin_bit_cast(half2_t, w);
-            f[2 * j] = (float)h.x;
-            f[2 * j + 1] = (float)h.y;
-        }
-    }
-};
-template <>
-struct Row8<float> {
-    float4 a, b;
-    __device__ __forceinline__ void load(const float* p) {
-        a = *reinterpret_cast<const float4*>(p);
-        b = *reinterpret_cast<const float4*>(p + 4);
-    }
-    __device__ __forceinline__ void get(float (&f)[8]) const {
-        f[0] = a.x, f[1] = a.y, f[2] = a.z, f[3] = a.w, f[4] = b.x, f[5] = b.y, f[6] = b.z, f[7] = b.w;
-    }
-};
-
 __device__ __forceinline__ float query_temperature(int pos, float coef, float every) {
     // (the quotient of two integers below 2^24 does not round up to the next one)
     return coef == 0.f ? 1.f : fmaf(coef, logf(floorf((float)(pos + 1) / every) + 1.0f), 1.0f);
@@ -109,27 +77,6 @@ __device__ __forceinline__ void block_sum2(float& a, float& b, float* red) {
     __syncthreads();
     a = b = 0.f;
     for (int i = 0; i < nw; i++) a += red[i], b += red[nw + i];
-}
-
-// the value of lane ^ OFF (8, 16 or 32), for sums and maxima over lanes that differ in that bit: f(v, other)
-template <int OFF, typename F>
-__device__ __forceinline__ float with_lane_xor(float v, F f) {
-    if constexpr (OFF == 8) return f(v, __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x128, 0xF, 0xF, true)));  // row rotated by 8
-    else if constexpr (OFF == 16) {
-        const auto r = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
-        return f(__uint_as_float(r[0]), __uint_as_float(r[1]));
-    } else {
-        const auto r = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
-        return f(__uint_as_float(r[0]), __uint_as_float(r[1]));
-    }
-}
-
-// over the 64 / LPT groups of a wavefront
-template <int LPT, typename F>
-__device__ __forceinline__ float over_groups(float v, F f) {
-    if constexpr (LPT <= 8) v = with_lane_xor<8>(v, f);
-    if constexpr (LPT <= 16) v = with_lane_xor<16>(v, f);
-    return with_lane_xor<32>(v, f);
 }
 
 // grid (splits, kv heads x head groups, query rows)
@@ -388,7 +335,7 @@ AttnArgs base_args(const skn_kv* kv, int seq, const skn_shared_attn& p) {
 }
 
 int check(skn_ctx* ctx, const skn_kv* kv, const skn_shared_attn& p) {
-    SKN_REQUIRE(ctx, kv->shared, SKN_ERR_STATE, "shared attention: the cache keeps keys and values apart");
+    SKN_REQUIRE(ctx, kv->kind == SKN_KV_SHARED, SKN_ERR_STATE, "shared attention: the cache keeps keys and values apart");
     SKN_REQUIRE(ctx, p.n_head > 0 && p.n_head % kv->n_head == 0, SKN_ERR_SHAPE, "shared attention: %d query heads over %d cached heads", p.n_head, kv->n_head);
     SKN_REQUIRE(ctx, p.q_norm && p.k_norm && (p.temp_coef == 0.f || p.temp_every > 0.f), SKN_ERR_ARG, "shared attention: bad parameters");
     return SKN_OK;

@@ -17,34 +17,13 @@
 // so S and Y are multiplied as they stand -- and no LDS, no barrier: a chunk's operands are coalesced loads one chunk ahead.
 // (Decays enter the triangles as ratios of products over at most sixteen tokens: any decay from 0.01 to 1 is safe in fp32.)
 // A decode step is one launch, one workgroup per head: the decay's low-rank product, the step, the head's norm and the gate.
+#include "delta.h"
 #include "dense.h"
 #include "rstate.h"
 
 #include <algorithm>
 
 namespace {
-
-constexpr float kUnitEps = 1e-6f;
-
-struct Vec8 {
-    float v[8];
-    __device__ __forceinline__ void load(const float* p) {
-        const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
-        v[0] = a.x, v[1] = a.y, v[2] = a.z, v[3] = a.w, v[4] = b.x, v[5] = b.y, v[6] = b.z, v[7] = b.w;
-    }
-    __device__ __forceinline__ void store(float* p) const {
-        *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
-        *reinterpret_cast<float4*>(p + 4) = make_float4(v[4], v[5], v[6], v[7]);
-    }
-};
-
-template <int L>
-__device__ __forceinline__ float dot_over_lanes(const Vec8& a, const Vec8& s) {
-    float x = a.v[0] * s.v[0], y = a.v[1] * s.v[1];
-#pragma unroll
-    for (int j = 2; j < 8; j += 2) x = fmaf(a.v[j], s.v[j], x), y = fmaf(a.v[j + 1], s.v[j + 1], y);
-    return lane_group_sum<L>(x + y);
-}
 
 // one token on one column; returns the column's output
 template <int L>
@@ -55,9 +34,6 @@ __device__ __forceinline__ float delta_column(Vec8& s, const Vec8& k, const Vec8
     return dot_over_lanes<L>(r, s);
 }
 
-typedef float f32x4 __attribute__((ext_vector_type(4)));
-
-constexpr int kChunk = 16;
 constexpr int kTrash = 64;  // floats behind the operands that take the outputs of tokens past the end
 
 // Operands of a chunk and head, in floats from its start.  Row operands (K1, R1: [token][channel], in tiles of 16 channels;
@@ -72,9 +48,6 @@ __host__ __device__ constexpr int off_a1(int dp) { return 80 * dp; }
 __host__ __device__ constexpr int off_g1(int dp) { return 80 * dp + 256; }
 __host__ __device__ constexpr int off_w(int dp) { return 80 * dp + 512; }
 __host__ __device__ constexpr int chunk_floats(int dp) { return 81 * dp + 512; }
-
-__device__ __forceinline__ f32x4 mma(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
-__device__ __forceinline__ f32x4 load4(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
 
 // N sums over the wavefront, step by step for all of them
 template <int N>
@@ -430,9 +403,9 @@ int launch_step(skn_ctx* ctx, const skn_rstate* st, const skn_delta_step& p, flo
     return SKN_OK;
 }
 
-__global__ void fill_zero_kernel(float4* p, int64_t n) {
+__global__ void fill_zero_kernel(float* p, int64_t n) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
-    if (i < n) p[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (i < n) p[i] = 0.f;
 }
 
 }  // namespace
@@ -472,22 +445,29 @@ int skn_delta_step_launch(skn_ctx* ctx, skn_rstate* st, int seq, const skn_delta
 
 extern "C" {
 
-int skn_rstate_create(skn_ctx* ctx, int n_seq, int heads, int dim, skn_rstate** out) {
+static int rstate_create(skn_ctx* ctx, int n_seq, int heads, int kv_heads, int dim, int vdim, int taps, skn_rstate** out) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_rstate_create: ctx is null");
     SKN_REQUIRE(ctx, out != nullptr, SKN_ERR_ARG, "skn_rstate_create: out is null");
     *out = nullptr;
     SKN_REQUIRE(ctx, n_seq > 0 && heads > 0, SKN_ERR_ARG, "skn_rstate_create: sizes must be positive");
-    SKN_REQUIRE(ctx, dim > 0 && dim <= 256, SKN_ERR_SHAPE, "skn_rstate_create: heads of %d channels (1 to 256)", dim);
+    SKN_REQUIRE(ctx, dim > 0 && dim <= 256 && vdim > 0 && vdim <= 256, SKN_ERR_SHAPE, "skn_rstate_create: heads of %d and %d channels (1 to 256)", dim, vdim);
     skn_rstate* st = new (std::nothrow) skn_rstate();
     SKN_REQUIRE(ctx, st != nullptr, SKN_ERR_OOM, "skn_rstate_create: host allocation failed");
     st->n_seq = n_seq;
     st->heads = heads;
     st->dim = dim;
+    st->vdim = vdim;
     st->dim_pad = dim <= 32 ? 32 : dim <= 64 ? 64 : dim <= 128 ? 128 : 256;
-    const size_t bytes = (size_t)n_seq * heads * dim * st->dim_pad * sizeof(float);
+    st->kv_heads = kv_heads;
+    st->taps = taps;
+    st->channels = 2 * kv_heads * dim + heads * vdim;
+    st->pos.assign(n_seq, 0);
+    const size_t bytes = (size_t)n_seq * heads * vdim * st->dim_pad * sizeof(float);
     hipError_t e = hipMalloc((void**)&st->s, bytes);
+    if (e == hipSuccess && taps > 0) e = hipMalloc((void**)&st->conv, (size_t)n_seq * taps * st->channels * sizeof(float));
     if (e != hipSuccess) {
         (void)hipGetLastError();
+        if (st->s) (void)hipFree(st->s);
         delete st;
         return skn_fail(ctx, SKN_ERR_OOM, "skn_rstate_create: %zu bytes: %s", bytes, hipGetErrorString(e));
     }
@@ -500,11 +480,23 @@ int skn_rstate_create(skn_ctx* ctx, int n_seq, int heads, int dim, skn_rstate** 
     return rc;
 }
 
+int skn_rstate_create(skn_ctx* ctx, int n_seq, int heads, int dim, skn_rstate** out) {
+    return rstate_create(ctx, n_seq, heads, 0, dim, dim, 0, out);
+}
+
+int skn_rstate_create_conv(skn_ctx* ctx, int n_seq, int heads, int kv_heads, int dim, int vdim, int taps, skn_rstate** out) {
+    SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_rstate_create_conv: ctx is null");
+    SKN_REQUIRE(ctx, heads > 0 && kv_heads > 0 && heads % kv_heads == 0, SKN_ERR_SHAPE, "skn_rstate_create_conv: kv_heads (%d) must divide heads (%d)", kv_heads, heads);
+    SKN_REQUIRE(ctx, taps >= 1 && taps <= 8, SKN_ERR_SHAPE, "skn_rstate_create_conv: convolutions of %d taps (1 to 8)", taps);
+    return rstate_create(ctx, n_seq, heads, kv_heads, dim, vdim, taps, out);
+}
+
 int skn_rstate_free(skn_ctx* ctx, skn_rstate* st) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_rstate_free: ctx is null");
     if (!st) return SKN_OK;
     (void)hipStreamSynchronize(ctx->stream);
     if (st->s) (void)hipFree(st->s);
+    if (st->conv) (void)hipFree(st->conv);
     delete st;
     return SKN_OK;
 }
@@ -513,9 +505,15 @@ int skn_rstate_reset(skn_ctx* ctx, skn_rstate* st, int seq) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_rstate_reset: ctx is null");
     SKN_REQUIRE(ctx, st != nullptr, SKN_ERR_ARG, "skn_rstate_reset: state is null");
     SKN_REQUIRE(ctx, seq >= -1 && seq < st->n_seq, SKN_ERR_RANGE, "skn_rstate_reset: sequence %d of %d", seq, st->n_seq);
-    const int64_t quads = (int64_t)st->heads * st->dim * st->dim_pad / 4 * (seq < 0 ? st->n_seq : 1);
-    skn_launch(ctx, fill_zero_kernel, dim3((unsigned)((quads + 255) / 256)), dim3(256), 0, (float4*)st->seq_state(seq < 0 ? 0 : seq), quads);
+    const int first = seq < 0 ? 0 : seq, count = seq < 0 ? st->n_seq : 1;
+    const int64_t n = (int64_t)st->heads * st->vdim * st->dim_pad * count, m = (int64_t)st->taps * st->channels * count;
+    skn_launch(ctx, fill_zero_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st->seq_state(first), n);
     SKN_LAUNCH_CHECK(ctx);
+    if (m > 0) {
+        skn_launch(ctx, fill_zero_kernel, dim3((unsigned)((m + 255) / 256)), dim3(256), 0, st->seq_conv(first), m);
+        SKN_LAUNCH_CHECK(ctx);
+    }
+    std::fill(st->pos.begin() + first, st->pos.begin() + first + count, 0);
     return SKN_OK;
 }
 
@@ -524,6 +522,7 @@ int skn_delta_rule(skn_ctx* ctx, skn_rstate* st, int seq, const float* r_dev, co
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_delta_rule: ctx is null");
     SKN_REQUIRE(ctx, st && r_dev && k_dev && v_dev && w_dev && a_dev && out_dev, SKN_ERR_ARG, "skn_delta_rule: null pointer");
     SKN_REQUIRE(ctx, seq >= 0 && seq < st->n_seq && n > 0, SKN_ERR_RANGE, "skn_delta_rule: %d tokens of sequence %d of %d", n, seq, st->n_seq);
+    SKN_REQUIRE(ctx, st->taps == 0, SKN_ERR_STATE, "skn_delta_rule: the state has convolutions (skn_gated_delta)");
     float* pack = nullptr;
     SKN_HIP(ctx, hipMalloc((void**)&pack, skn_delta_pack_floats(st, n) * sizeof(float)));
     const int rc = skn_delta_rows(ctx, st, seq, r_dev, k_dev, v_dev, w_dev, a_dev, st->heads * st->dim, n, pack, out_dev);

@@ -35,6 +35,8 @@ struct Shape {
     static constexpr int kLds = ST * kBuf > kOutBytes ? ST * kBuf : kOutBytes;
 };
 
+__device__ __forceinline__ uint32_t half_bits(float f) { return __half_as_ushort(__float2half_rn(f)); }
+
 template <typename T>
 __device__ __forceinline__ float16_t mma(const u32x4& a, const u32x4& b, float16_t c) {
     if constexpr (std::is_same<T, float>::value) {
@@ -169,17 +171,24 @@ __global__ __launch_bounds__(S::kThreads) void dense_gemm_kernel(const uint8_t* 
             }
 #pragma unroll
             for (int e = 0; e < 4; e++) v[e] = skn_dense_op(sg.op, v[e], sg.p0, sg.p1);
+            if (si == out.mul_seg) {
+                const int64_t from = (int64_t)out.mul_tokens[t] * out.mul_ld + out.mul_col + (row - sg.row0);
+#pragma unroll
+                for (int e = 0; e < 4; e++) v[e] *= e < left ? skn_table_at(out.mul_table, out.mul_type, from + e) : 0.f;
+            }
             const int64_t at = (int64_t)t * sg.ldo + (row - sg.row0);
             if (left >= 4 && sg.out_type == SKN_TYPE_F32) {
                 *reinterpret_cast<float4*>((float*)sg.out + at) = make_float4(v[0], v[1], v[2], v[3]);
             } else if (left >= 4) {
-                *reinterpret_cast<uint2*>((uint16_t*)sg.out + at) = make_uint2(skn_bf16_bits(v[0]) | ((uint32_t)skn_bf16_bits(v[1]) << 16),
+                if (sg.out_type == SKN_TYPE_F16)
+                    *reinterpret_cast<uint2*>((uint16_t*)sg.out + at) = make_uint2(half_bits(v[0]) | (half_bits(v[1]) << 16), half_bits(v[2]) | (half_bits(v[3]) << 16));
+                else *reinterpret_cast<uint2*>((uint16_t*)sg.out + at) = make_uint2(skn_bf16_bits(v[0]) | ((uint32_t)skn_bf16_bits(v[1]) << 16),
                                                                                 skn_bf16_bits(v[2]) | ((uint32_t)skn_bf16_bits(v[3]) << 16));
             } else {
                 for (int e = 0; e < left; e++) {
                     const float f = e == 0 ? v[0] : e == 1 ? v[1] : v[2];
                     if (sg.out_type == SKN_TYPE_F32) ((float*)sg.out)[at + e] = f;
-                    else ((uint16_t*)sg.out)[at + e] = skn_bf16_bits(f);
+                    else ((uint16_t*)sg.out)[at + e] = sg.out_type == SKN_TYPE_F16 ? (uint16_t)half_bits(f) : skn_bf16_bits(f);
                 }
             }
         }
@@ -260,6 +269,7 @@ int skn_dense_gemm(skn_ctx* ctx, const skn_dense_mat& w, const void* a, int lda,
         SKN_REQUIRE(ctx, out.seg[i].out && out.seg[i].row0 % kDenseRowPad == 0 && out.seg[i].ldo % 4 == 0 && ((uintptr_t)out.seg[i].out & 15) == 0 &&
                              out.seg[i].row0 + skn_pad_rows(out.seg[i].rows) <= w.rows && (i == 0 || out.seg[i].row0 > out.seg[i - 1].row0),
                     SKN_ERR_ARG, "dense GEMM: segment %d is misplaced", i);
+    SKN_REQUIRE(ctx, out.mul_seg < 0 || (out.mul_table && out.mul_tokens), SKN_ERR_ARG, "dense GEMM: no table to multiply with");
     SKN_REQUIRE(ctx, out.nseg > 0 || (out.ldr % 4 == 0 && out.resid_rows <= w.rows && ((uintptr_t)out.resid & 15) == 0), SKN_ERR_ARG,
                 "dense GEMM: bad residual rows");
     if (w.type == SKN_TYPE_BF16) return pick_gemm<uint16_t>(ctx, w, a, lda, m, out);

@@ -79,6 +79,43 @@ __device__ __forceinline__ void stage_group_norm(const skn_matvec_src& s, const 
     for (int e = tid; e < s.k0; e += kThreads) xs.at(e) *= red[e / gs] * s.norm_w[e];
 }
 
+// the sum over the workgroup (a barrier inside; red: one float per wavefront, used once)
+__device__ __forceinline__ float block_sum(float v, float* red) {
+    v = wave_sum(v);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    v = 0.f;
+#pragma unroll
+    for (int i = 0; i < kWaves; i++) v += red[i];
+    return v;
+}
+
+// (pitches are multiples of 64 elements and their padding is zero, as in stage_group_norm; a thread's quads stay its own)
+__device__ __forceinline__ void stage_add_norm(const skn_matvec_src& s, const XPlanes& xs, float* red) {
+    const int tid = threadIdx.x, quads = (s.k0 + 3) >> 2;
+    auto square = [](const float4& v) { return (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w); };
+    float ss = 0.f;
+    for (int q = tid; q < quads; q += kThreads) {
+        const float4 v = reinterpret_cast<const float4*>(s.add)[q];
+        xs.quad(q) = v;
+        ss += square(v);
+    }
+    const float ry = 1.0f / sqrtf(block_sum(ss, red) / (float)s.k0 + s.eps);
+    ss = 0.f;
+    for (int q = tid; q < quads; q += kThreads) {
+        const float4 y = xs.quad(q), x = reinterpret_cast<const float4*>(s.x0)[q], g = reinterpret_cast<const float4*>(s.add_w)[q];
+        const float4 v = make_float4(fmaf(y.x * ry, g.x, x.x), fmaf(y.y * ry, g.y, x.y), fmaf(y.z * ry, g.z, x.z), fmaf(y.w * ry, g.w, x.w));
+        xs.quad(q) = v;
+        if (blockIdx.x == 0) reinterpret_cast<float4*>(s.x_out)[q] = v;
+        ss += square(v);
+    }
+    const float rx = 1.0f / sqrtf(block_sum(ss, red + kWaves) / (float)s.k0 + s.eps);
+    for (int q = tid; q < quads; q += kThreads) {
+        const float4 v = xs.quad(q), g = reinterpret_cast<const float4*>(s.norm_w)[q];
+        xs.quad(q) = make_float4(v.x * rx * g.x, v.y * rx * g.y, v.z * rx * g.z, v.w * rx * g.w);
+    }
+}
+
 // red: heads x splits weights
 __device__ __forceinline__ void stage_merge(const skn_matvec_src& s, const XPlanes& xs, float* red) {
     const int tid = threadIdx.x;
@@ -86,9 +123,10 @@ __device__ __forceinline__ void stage_merge(const skn_matvec_src& s, const XPlan
         float2 ml[kMaxSplits];  // (all requested before the first is used)
 #pragma unroll
         for (int i = 0; i < kMaxSplits; i++) ml[i] = reinterpret_cast<const float2*>(s.ml)[min(i, s.splits - 1) * s.heads + h];
-        float m = -INFINITY, l = 0.f;
+        float m = s.sink ? 0.f : -INFINITY;
 #pragma unroll
         for (int i = 0; i < kMaxSplits; i++) m = fmaxf(m, ml[i].x);
+        float l = s.sink ? __builtin_amdgcn_exp2f(-m) : 0.f;
 #pragma unroll
         for (int i = 0; i < kMaxSplits; i++) {
             ml[i].x = i < s.splits ? __builtin_amdgcn_exp2f(ml[i].x - m) : 0.f;  // (an empty split: exp2(-inf) = 0)
@@ -117,6 +155,10 @@ __device__ __forceinline__ void stage_merge(const skn_matvec_src& s, const XPlan
                     a.x = fmaf(f, v[i].x, a.x), a.y = fmaf(f, v[i].y, a.y), a.z = fmaf(f, v[i].z, a.z), a.w = fmaf(f, v[i].w, a.w);
                 }
             }
+            if (s.gate) {
+                const float4 g = reinterpret_cast<const float4*>(s.gate)[q];
+                a.x *= g.x, a.y *= g.y, a.z *= g.z, a.w *= g.w;
+            }
             xs.quad(q) = a;
         }
         return;
@@ -125,7 +167,7 @@ __device__ __forceinline__ void stage_merge(const skn_matvec_src& s, const XPlan
         const int h = e / s.dim, d = e - h * s.dim;
         float a = 0.f;
         for (int i = 0; i < s.splits; i++) a = fmaf(red[h * s.splits + i], s.x0[((int64_t)i * s.heads + h) * s.dim_pad + d], a);
-        xs.at(e) = a;
+        xs.at(e) = s.gate ? a * s.gate[e] : a;
     }
 }
 
@@ -156,6 +198,7 @@ __global__ __launch_bounds__(kThreads) void dense_matvec_kernel(const W* __restr
 
     // ---- staging ----
     if constexpr (MODE == SKN_XSRC_GROUP_NORM) stage_group_norm(src, xs, reinterpret_cast<float*>(lds4 + 2 * plane));
+    else if constexpr (MODE == SKN_XSRC_ADD_NORM) stage_add_norm(src, xs, reinterpret_cast<float*>(lds4 + 2 * plane));
     else if constexpr (MODE == SKN_XSRC_MERGE) stage_merge(src, xs, reinterpret_cast<float*>(lds4 + 2 * plane));
     else {
         for (int q = tid; q < src.k0 >> 2; q += kThreads) xs.quad(q) = reinterpret_cast<const float4*>(src.x0)[q];
@@ -167,7 +210,7 @@ __global__ __launch_bounds__(kThreads) void dense_matvec_kernel(const W* __restr
     }
     {
         const int gap_end = src.x1 ? src.off1 : 8 * plane, tail = src.x1 ? src.off1 + src.k1 : 8 * plane;
-        if constexpr (MODE == SKN_XSRC_GROUP_NORM) __syncthreads();  // (its last quad may have been written past k0)
+        if constexpr (MODE == SKN_XSRC_GROUP_NORM || MODE == SKN_XSRC_ADD_NORM) __syncthreads();  // (its last quad may have been written past k0)
         for (int e = src.k0 + tid; e < gap_end; e += kThreads) xs.at(e) = 0.f;
         for (int e = tail + tid; e < 8 * plane; e += kThreads) xs.at(e) = 0.f;
     }
@@ -182,6 +225,7 @@ __global__ __launch_bounds__(kThreads) void dense_matvec_kernel(const W* __restr
         cache_page = out.page_table[pos / out.page_tokens];
         cache_slot = pos % out.page_tokens;
     }
+    const int64_t mul_at = out.mul_seg >= 0 ? (int64_t)*out.mul_tokens * out.mul_ld + out.mul_col : 0;
     float acc[kR];
 #pragma unroll
     for (int r = 0; r < kR; r++) acc[r] = 0.f;
@@ -236,6 +280,7 @@ __global__ __launch_bounds__(kThreads) void dense_matvec_kernel(const W* __restr
         const int r = row - sg.row0;
         if (r >= sg.rows) return;
         z = skn_dense_op(sg.op, z, sg.p0, sg.p1);
+        if (si == out.mul_seg) z *= skn_table_at(out.mul_table, out.mul_type, mul_at + r);
         if (sg.out_type == SKN_TYPE_F32) ((float*)sg.out)[r] = z;
         else ((uint16_t*)sg.out)[r] = skn_bf16_bits(z);
         if (si == out.cache_seg) {
@@ -275,7 +320,7 @@ int launch(skn_ctx* ctx, const skn_dense_mat& w, const skn_matvec_src& src, cons
     constexpr int V = 16 / (int)sizeof(W);
     const int chunk = 64 * kU * V;  // elements of a turn: the planes hold whole turns
     const int plane = (w.k_pad + chunk - 1) / chunk * chunk / 8;
-    const size_t scratch = MODE == SKN_XSRC_GROUP_NORM ? (kMaxGroups + 16 * kWaves) * 4 : MODE == SKN_XSRC_MERGE ? (size_t)src.heads * src.splits * 4 : 0;
+    const size_t scratch = MODE == SKN_XSRC_GROUP_NORM || MODE == SKN_XSRC_ADD_NORM ? (kMaxGroups + 16 * kWaves) * 4 : MODE == SKN_XSRC_MERGE ? (size_t)src.heads * src.splits * 4 : 0;
     const size_t lds = (size_t)plane * 32 + scratch;
     SKN_REQUIRE(ctx, lds <= kMaxLds, SKN_ERR_SHAPE, "dense matvec: %d columns need %zu bytes of LDS (at most %d)", w.k_pad, lds, kMaxLds);
     // one workgroup per compute unit at most: its staging serves all the rows its wavefronts walk through
@@ -288,6 +333,7 @@ int launch(skn_ctx* ctx, const skn_dense_mat& w, const skn_matvec_src& src, cons
 template <typename W>
 int launch_mode(skn_ctx* ctx, const skn_dense_mat& w, const skn_matvec_src& src, const skn_dense_out& out) {
     if (src.mode == SKN_XSRC_GROUP_NORM) return launch<W, SKN_XSRC_GROUP_NORM>(ctx, w, src, out);
+    if (src.mode == SKN_XSRC_ADD_NORM) return launch<W, SKN_XSRC_ADD_NORM>(ctx, w, src, out);
     if (src.mode == SKN_XSRC_MERGE) return launch<W, SKN_XSRC_MERGE>(ctx, w, src, out);
     return launch<W, SKN_XSRC_PLAIN>(ctx, w, src, out);
 }
@@ -301,7 +347,9 @@ int allow_lds(skn_ctx* ctx) {
 int dense_matvec_init(skn_ctx* ctx) {
     SKN_TRY((allow_lds<uint16_t, SKN_XSRC_PLAIN>(ctx)));
     SKN_TRY((allow_lds<uint16_t, SKN_XSRC_GROUP_NORM>(ctx)));
+    SKN_TRY((allow_lds<uint16_t, SKN_XSRC_ADD_NORM>(ctx)));
     SKN_TRY((allow_lds<uint16_t, SKN_XSRC_MERGE>(ctx)));
+    SKN_TRY((allow_lds<float, SKN_XSRC_ADD_NORM>(ctx)));
     SKN_TRY((allow_lds<float, SKN_XSRC_PLAIN>(ctx)));
     SKN_TRY((allow_lds<float, SKN_XSRC_GROUP_NORM>(ctx)));
     return allow_lds<float, SKN_XSRC_MERGE>(ctx);
@@ -318,6 +366,9 @@ int skn_dense_matvec(skn_ctx* ctx, const skn_dense_mat& w, const skn_matvec_src&
                 "dense matvec: bad second input");
     SKN_REQUIRE(ctx, src.mode != SKN_XSRC_GROUP_NORM || (src.norm_w && src.groups > 0 && src.groups <= kMaxGroups && src.k0 % src.groups == 0),
                 SKN_ERR_SHAPE, "dense matvec: %d norm groups of %d columns (at most %d groups)", src.groups, src.k0, kMaxGroups);
+    SKN_REQUIRE(ctx, src.mode != SKN_XSRC_ADD_NORM || (src.norm_w && src.add && src.add_w && src.x_out && src.x_out != src.x0), SKN_ERR_ARG,
+                "dense matvec: a sum and norm without its vectors");
+    SKN_REQUIRE(ctx, out.mul_seg < 0 || (out.mul_table && out.mul_tokens), SKN_ERR_ARG, "dense matvec: no table to multiply with");
     SKN_REQUIRE(ctx, src.mode != SKN_XSRC_MERGE || (src.ml && src.splits > 0 && src.splits <= kMaxSplits && src.heads * src.splits <= kMaxMerge && src.k0 == src.heads * src.dim &&
                                                      src.dim_pad % 4 == 0),
                 SKN_ERR_SHAPE, "dense matvec: cannot merge %d heads x %d splits", src.heads, src.splits);

@@ -1,4 +1,5 @@
-// Row-wise kernels around the dense products: RMS norm in groups, and the embedding with sinusoidal positions.
+// Row-wise kernels around the dense products: RMS norm in groups, the sum of a normed row with the norm that follows, and the
+// embedding, scaled or with sinusoidal positions.
 #include "dense.h"
 
 namespace {
@@ -45,28 +46,75 @@ __global__ __launch_bounds__(256) void group_norm_kernel(const float* __restrict
 }
 
 // The angle is formed and reduced modulo 2 pi in double (as the rotary embedding's is).
-__global__ __launch_bounds__(256) void embed_sinusoid_kernel(const void* __restrict__ table, int table_type, int ld_table,
-                                                             const int32_t* __restrict__ tokens, const int32_t* __restrict__ pos0_dev,
-                                                             const double* __restrict__ inv_freq, int width, float* __restrict__ x, int ldx) {
+__global__ __launch_bounds__(256) void embed_kernel(const void* __restrict__ table, int table_type, int ld_table,
+                                                    const int32_t* __restrict__ tokens, const int32_t* __restrict__ pos0_dev,
+                                                    const double* __restrict__ inv_freq, float scale, int width, float* __restrict__ x, int ldx) {
     const int row = blockIdx.x, pos = pos0_dev[0] + row;
     const int64_t at = (int64_t)tokens[row] * ld_table;
     for (int i = blockIdx.y * 256 + threadIdx.x; 2 * i < width; i += gridDim.y * 256) {
-        float sn, cs;
-        skn_rope_sincos_freq(pos, inv_freq[i], &sn, &cs);
+        float sn = 0.f, cs = 0.f;
+        if (inv_freq) skn_rope_sincos_freq(pos, inv_freq[i], &sn, &cs);
 #pragma unroll
         for (int e = 0; e < 2; e++) {
             const int col = 2 * i + e;
             if (col >= width) continue;
-            const float v = table_type == SKN_TYPE_F32 ? ((const float*)table)[at + col]
-                                                       : __uint_as_float((uint32_t)((const uint16_t*)table)[at + col] << 16);
-            x[(int64_t)row * ldx + col] = v + (e ? cs : sn);
+            x[(int64_t)row * ldx + col] = fmaf(scale, skn_table_at(table, table_type, at + col), e ? cs : sn);
         }
     }
+}
+
+// one workgroup per row; LDS: the row
+__global__ __launch_bounds__(256) void add_norm_kernel(float* __restrict__ x, int ldx, const float* __restrict__ y, int ldy, const float* __restrict__ y_w,
+                                                       const float* __restrict__ w, int width, float eps, void* __restrict__ h, int ldh, int h_type) {
+    extern __shared__ float lds[];
+    __shared__ float part[8];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    float* xr = x + (int64_t)blockIdx.x * ldx;
+    const float* yr = y + (int64_t)blockIdx.x * ldy;
+    auto inv_rms = [&](float ss, float* red) {
+        ss = wave_sum(ss);
+        if (lane == 0) red[wave] = ss;
+        __syncthreads();
+        return 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)width + eps);
+    };
+    float ss = 0.f;
+    for (int i = tid; i < width; i += 256) {
+        const float v = yr[i];
+        lds[i] = v;
+        ss = fmaf(v, v, ss);
+    }
+    const float ry = inv_rms(ss, part);
+    ss = 0.f;
+    for (int i = tid; i < width; i += 256) {  // (a thread's own elements throughout)
+        const float v = xr[i] + lds[i] * ry * y_w[i];
+        xr[i] = v;
+        lds[i] = v;
+        ss = fmaf(v, v, ss);
+    }
+    if (!w) return;
+    const float rx = inv_rms(ss, part + 4);
+    for (int i = tid; i < ldh; i += 256) {
+        const float v = i < width ? lds[i] * rx * w[i] : 0.f;
+        if (h_type == SKN_TYPE_F32) ((float*)h)[(int64_t)blockIdx.x * ldh + i] = v;
+        else ((uint16_t*)h)[(int64_t)blockIdx.x * ldh + i] = skn_bf16_bits(v);
+    }
+}
+
+__global__ __launch_bounds__(256) void bf16_rows_kernel(const float4* __restrict__ x, int64_t n, uint2* __restrict__ y) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n) return;
+    const float4 v = x[i];
+    y[i] = make_uint2(skn_bf16_bits(v.x) | ((uint32_t)skn_bf16_bits(v.y) << 16), skn_bf16_bits(v.z) | ((uint32_t)skn_bf16_bits(v.w) << 16));
 }
 
 __global__ void xielu_kernel(const float* __restrict__ z, int64_t n, float p0, float p1, float* __restrict__ out) {
     const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i < n) out[i] = skn_xielu_at(z[i], p0, p1);
+}
+
+__global__ void gelu_kernel(const float* __restrict__ z, int64_t n, float* __restrict__ out) {
+    const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) out[i] = skn_dense_op(SKN_OP_GELU, z[i], 0.f, 0.f);
 }
 
 }  // namespace
@@ -82,11 +130,27 @@ int skn_group_norm_rows(skn_ctx* ctx, const float* x, int ldx, const int32_t* ro
     return SKN_OK;
 }
 
-int skn_embed_sinusoid_rows(skn_ctx* ctx, const void* table, int table_type, int ld_table, const int32_t* tokens, const int32_t* pos0_dev,
-                            const double* inv_freq, int n_rows, int width, float* x, int ldx) {
+int skn_add_norm_rows(skn_ctx* ctx, float* x, int ldx, const float* y, int ldy, const float* y_w, const float* w, int n_rows, int width, float eps,
+                      void* h, int ldh, int h_type) {
+    SKN_REQUIRE(ctx, width > 0 && width <= 16000, SKN_ERR_SHAPE, "norm: rows of %d columns (at most 16000)", width);
+    skn_launch(ctx, add_norm_kernel, dim3(n_rows), dim3(256), (size_t)width * sizeof(float), x, ldx, y, ldy, y_w, w, width, eps, h, ldh, h_type);
+    SKN_LAUNCH_CHECK(ctx);
+    return SKN_OK;
+}
+
+int skn_bf16_rows(skn_ctx* ctx, const float* x, int ld, int n_rows, void* y) {
+    SKN_REQUIRE(ctx, ld % 4 == 0, SKN_ERR_SHAPE, "bf16 rows: pitch %d is no multiple of 4", ld);
+    const int64_t quads = (int64_t)n_rows * ld / 4;
+    skn_launch(ctx, bf16_rows_kernel, dim3((unsigned)((quads + 255) / 256)), dim3(256), 0, (const float4*)x, quads, (uint2*)y);
+    SKN_LAUNCH_CHECK(ctx);
+    return SKN_OK;
+}
+
+int skn_embed_rows(skn_ctx* ctx, const void* table, int table_type, int ld_table, const int32_t* tokens, const int32_t* pos0_dev,
+                   const double* inv_freq, float scale, int n_rows, int width, float* x, int ldx) {
     // (a single row: its columns over several workgroups)
     const int split = n_rows == 1 ? (width + 511) / 512 : 1;
-    skn_launch(ctx, embed_sinusoid_kernel, dim3(n_rows, split), dim3(256), 0, table, table_type, ld_table, tokens, pos0_dev, inv_freq, width, x, ldx);
+    skn_launch(ctx, embed_kernel, dim3(n_rows, split), dim3(256), 0, table, table_type, ld_table, tokens, pos0_dev, inv_freq, scale, width, x, ldx);
     SKN_LAUNCH_CHECK(ctx);
     return SKN_OK;
 }
@@ -107,6 +171,16 @@ int skn_xielu(skn_ctx* ctx, const float* z_dev, int64_t n, float pos, float neg,
     if (n == 0) return SKN_OK;
     SKN_REQUIRE(ctx, z_dev && out_dev, SKN_ERR_ARG, "skn_xielu: null pointer");
     skn_launch(ctx, xielu_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, z_dev, n, pos, neg, out_dev);
+    SKN_LAUNCH_CHECK(ctx);
+    return SKN_OK;
+}
+
+int skn_gelu(skn_ctx* ctx, const float* z_dev, int64_t n, float* out_dev) {
+    SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_gelu: ctx is null");
+    SKN_REQUIRE(ctx, n >= 0, SKN_ERR_ARG, "skn_gelu: negative size");
+    if (n == 0) return SKN_OK;
+    SKN_REQUIRE(ctx, z_dev && out_dev, SKN_ERR_ARG, "skn_gelu: null pointer");
+    skn_launch(ctx, gelu_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, z_dev, n, out_dev);
     SKN_LAUNCH_CHECK(ctx);
     return SKN_OK;
 }

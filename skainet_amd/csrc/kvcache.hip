@@ -124,7 +124,15 @@ int skn_kv_advance_len(skn_ctx* ctx, skn_kv* kv, int seq, int n) {
 
 extern "C" {
 
-static int kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page_tokens, int max_tokens, bool shared, int elem_type, int dim,
+static int padded_head(int dim) { return dim <= 64 ? 64 : dim <= 128 ? 128 : 256; }
+
+static int check_padded(skn_ctx* ctx, const char* who, int elem_type, int max_tokens) {
+    SKN_REQUIRE(ctx, elem_type == SKN_TYPE_F16 || elem_type == SKN_TYPE_F32, SKN_ERR_TYPE, "%s: type %d (F16 or F32)", who, elem_type);
+    SKN_REQUIRE(ctx, max_tokens <= 1 << 22, SKN_ERR_SHAPE, "%s: %d tokens (at most %d)", who, max_tokens, 1 << 22);
+    return SKN_OK;
+}
+
+static int kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page_tokens, int max_tokens, int kind, int elem_type, int dim, int vdim,
                      skn_kv** out) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_create: ctx is null");
     SKN_REQUIRE(ctx, out != nullptr, SKN_ERR_ARG, "skn_kv_create: out is null");
@@ -137,9 +145,10 @@ static int kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page
     kv->n_seq = n_seq;
     kv->n_head = n_head;
     kv->head_dim = head_dim;
-    kv->shared = shared;
+    kv->kind = kind;
     kv->elem_type = elem_type;
     kv->dim = dim;
+    kv->vdim = vdim;
     kv->page_tokens = page_tokens;
     kv->max_tokens = max_tokens;
     kv->pages_per_seq = (max_tokens + page_tokens - 1) / page_tokens;
@@ -149,8 +158,8 @@ static int kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page
     const size_t scale_bytes = (size_t)kv->n_pages * page_tokens * sizeof(float);
     const size_t table_bytes = (size_t)n_seq * kv->pages_per_seq * sizeof(int32_t);
     hipError_t e = hipMalloc((void**)&kv->k_pool, pool_bytes);
-    if (e == hipSuccess && !shared) e = hipMalloc((void**)&kv->v_pool, pool_bytes);
-    if (e == hipSuccess && shared) e = hipMalloc((void**)&kv->key_scale, scale_bytes);
+    if (e == hipSuccess && (kind == SKN_KV_PLAIN || kind == SKN_KV_RANGED)) e = hipMalloc((void**)&kv->v_pool, pool_bytes);
+    if (e == hipSuccess && kind == SKN_KV_SHARED) e = hipMalloc((void**)&kv->key_scale, scale_bytes);
     if (e == hipSuccess) e = hipMalloc((void**)&kv->page_table_dev, table_bytes);
     if (e == hipSuccess) e = hipMalloc((void**)&kv->len_dev, (size_t)n_seq * sizeof(int32_t));
     if (e == hipSuccess) e = hipMalloc((void**)&kv->nctx_dev, (size_t)n_seq * sizeof(int32_t));
@@ -169,9 +178,10 @@ static int kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page
     if (rc == SKN_OK) rc = skn_memset(ctx, kv->len_dev, 0, (size_t)n_seq * sizeof(int32_t));
     if (rc == SKN_OK) rc = skn_memset(ctx, kv->nctx_dev, 0, (size_t)n_seq * sizeof(int32_t));
     if (rc == SKN_OK) rc = skn_memset(ctx, kv->ticket_dev, 0, 16);
-    // (the kernels of a shared cache read its rows up to head_dim: what no token writes is zero)
-    if (rc == SKN_OK && shared) rc = skn_memset(ctx, kv->k_pool, 0, pool_bytes);
-    if (rc == SKN_OK && shared) rc = skn_memset(ctx, kv->key_scale, 0, scale_bytes);
+    // (the kernels read padded rows up to head_dim: what no token writes is zero)
+    if (rc == SKN_OK && kind != SKN_KV_PLAIN) rc = skn_memset(ctx, kv->k_pool, 0, pool_bytes);
+    if (rc == SKN_OK && kind == SKN_KV_RANGED) rc = skn_memset(ctx, kv->v_pool, 0, pool_bytes);
+    if (rc == SKN_OK && kv->key_scale) rc = skn_memset(ctx, kv->key_scale, 0, scale_bytes);
     if (rc != SKN_OK) {
         skn_kv_free(ctx, kv);
         return rc;
@@ -181,15 +191,30 @@ static int kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page
 }
 
 int skn_kv_create(skn_ctx* ctx, int n_seq, int n_head, int head_dim, int page_tokens, int max_tokens, skn_kv** out) {
-    return kv_create(ctx, n_seq, n_head, head_dim, page_tokens, max_tokens, false, SKN_TYPE_F16, head_dim, out);
+    return kv_create(ctx, n_seq, n_head, head_dim, page_tokens, max_tokens, SKN_KV_PLAIN, SKN_TYPE_F16, head_dim, head_dim, out);
 }
 
 int skn_kv_create_shared(skn_ctx* ctx, int n_seq, int n_head, int dim, int elem_type, int page_tokens, int max_tokens, skn_kv** out) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_create_shared: ctx is null");
     SKN_REQUIRE(ctx, dim > 0 && dim <= 256, SKN_ERR_SHAPE, "skn_kv_create_shared: heads of %d elements (1 to 256)", dim);
-    SKN_REQUIRE(ctx, elem_type == SKN_TYPE_F16 || elem_type == SKN_TYPE_F32, SKN_ERR_TYPE, "skn_kv_create_shared: type %d (F16 or F32)", elem_type);
-    SKN_REQUIRE(ctx, max_tokens <= 1 << 22, SKN_ERR_SHAPE, "skn_kv_create_shared: %d tokens (at most %d)", max_tokens, 1 << 22);
-    return kv_create(ctx, n_seq, n_head, dim <= 64 ? 64 : dim <= 128 ? 128 : 256, page_tokens, max_tokens, true, elem_type, dim, out);
+    SKN_TRY(check_padded(ctx, "skn_kv_create_shared", elem_type, max_tokens));
+    return kv_create(ctx, n_seq, n_head, padded_head(dim), page_tokens, max_tokens, SKN_KV_SHARED, elem_type, dim, dim, out);
+}
+
+int skn_kv_create_ranged(skn_ctx* ctx, int n_seq, int n_head, int dim, int vdim, int elem_type, int page_tokens, int max_tokens, skn_kv** out) {
+    SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_create_ranged: ctx is null");
+    SKN_REQUIRE(ctx, dim > 0 && dim <= 256 && vdim > 0 && vdim <= 256, SKN_ERR_SHAPE, "skn_kv_create_ranged: keys of %d and values of %d elements (1 to 256)", dim, vdim);
+    SKN_TRY(check_padded(ctx, "skn_kv_create_ranged", elem_type, max_tokens));
+    return kv_create(ctx, n_seq, n_head, padded_head(dim > vdim ? dim : vdim), page_tokens, max_tokens, SKN_KV_RANGED, elem_type, dim, vdim, out);
+}
+
+int skn_kv_create_latent(skn_ctx* ctx, int n_seq, int rank, int rot_dim, int elem_type, int page_tokens, int max_tokens, skn_kv** out) {
+    SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_create_latent: ctx is null");
+    SKN_REQUIRE(ctx, rank > 0 && rot_dim >= 0 && rot_dim % 2 == 0 && rot_dim <= 256 && rank + rot_dim <= 1024, SKN_ERR_SHAPE,
+                "skn_kv_create_latent: latents of %d and rotated keys of %d elements (together at most 1024, the latter even and at most 256)", rank, rot_dim);
+    SKN_TRY(check_padded(ctx, "skn_kv_create_latent", elem_type, max_tokens));
+    const int w = rank + rot_dim, pieces = (w + 127) / 128;
+    return kv_create(ctx, n_seq, 1, 128 * (pieces <= 3 ? pieces : pieces <= 5 ? 5 : 8), page_tokens, max_tokens, SKN_KV_LATENT, elem_type, w, rank, out);
 }
 
 int skn_kv_free(skn_ctx* ctx, skn_kv* kv) {
@@ -231,7 +256,7 @@ int skn_kv_append(skn_ctx* ctx, skn_kv* kv, const uint16_t* k_dev, const uint16_
                   int n) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_append: ctx is null");
     SKN_REQUIRE(ctx, kv != nullptr, SKN_ERR_ARG, "skn_kv_append: kv is null");
-    SKN_REQUIRE(ctx, !kv->shared, SKN_ERR_STATE, "skn_kv_append: the cache shares its keys and values");
+    SKN_REQUIRE(ctx, kv->kind == SKN_KV_PLAIN, SKN_ERR_STATE, "skn_kv_append: not a cache of fp16 keys and values");
     SKN_REQUIRE(ctx, n >= 0, SKN_ERR_ARG, "skn_kv_append: negative count");
     if (n == 0) return SKN_OK;
     SKN_REQUIRE(ctx, k_dev && v_dev && seq_ids_host, SKN_ERR_ARG, "skn_kv_append: null pointer");
@@ -273,7 +298,7 @@ int skn_kv_append(skn_ctx* ctx, skn_kv* kv, const uint16_t* k_dev, const uint16_
 int skn_kv_append_run(skn_ctx* ctx, skn_kv* kv, int seq, const uint16_t* k_dev, const uint16_t* v_dev, int n_tokens) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_append_run: ctx is null");
     SKN_REQUIRE(ctx, kv != nullptr, SKN_ERR_ARG, "skn_kv_append_run: kv is null");
-    SKN_REQUIRE(ctx, !kv->shared, SKN_ERR_STATE, "skn_kv_append_run: the cache shares its keys and values");
+    SKN_REQUIRE(ctx, kv->kind == SKN_KV_PLAIN, SKN_ERR_STATE, "skn_kv_append_run: not a cache of fp16 keys and values");
     SKN_REQUIRE(ctx, seq >= 0 && seq < kv->n_seq, SKN_ERR_RANGE, "skn_kv_append_run: sequence %d of %d", seq, kv->n_seq);
     SKN_REQUIRE(ctx, n_tokens >= 0, SKN_ERR_ARG, "skn_kv_append_run: negative count");
     if (n_tokens == 0) return SKN_OK;
@@ -297,7 +322,7 @@ int skn_kv_append_run(skn_ctx* ctx, skn_kv* kv, int seq, const uint16_t* k_dev, 
 int skn_kv_gather(skn_ctx* ctx, skn_kv* kv, int seq, int t0, int t1, uint16_t* k_out_dev, uint16_t* v_out_dev) {
     SKN_REQUIRE(nullptr, ctx != nullptr, SKN_ERR_ARG, "skn_kv_gather: ctx is null");
     SKN_REQUIRE(ctx, kv != nullptr, SKN_ERR_ARG, "skn_kv_gather: kv is null");
-    SKN_REQUIRE(ctx, !kv->shared, SKN_ERR_STATE, "skn_kv_gather: the cache shares its keys and values");
+    SKN_REQUIRE(ctx, kv->kind == SKN_KV_PLAIN, SKN_ERR_STATE, "skn_kv_gather: not a cache of fp16 keys and values");
     SKN_REQUIRE(ctx, seq >= 0 && seq < kv->n_seq, SKN_ERR_RANGE, "skn_kv_gather: sequence %d of %d", seq, kv->n_seq);
     SKN_REQUIRE(ctx, t0 >= 0 && t0 <= t1 && t1 <= kv->len[seq], SKN_ERR_RANGE,
                 "skn_kv_gather: tokens [%d, %d) of a sequence holding %d", t0, t1, kv->len[seq]);

@@ -13,6 +13,7 @@ import os
 ARCHITECTURES = {
     "llama": ("skainet_amd.llama", "load"),
     "Nusilix": ("skainet_amd.nusilix", "load"),
+    "Lebelix": ("skainet_amd.lebelix", "load"),
 }
 
 

@@ -7,20 +7,15 @@ csrc/delta.hip).  Feed-forward: xIELU between two matrices, or none.
 """
 from __future__ import annotations
 
-import ctypes as C
-import json
-import os
 from dataclasses import dataclass, field
 
 import numpy as np
 
 from . import runtime
-from .decoder import DecoderModel
-from .runtime import BF16, F32, HybridConfig, HybridLayer, HybridWeights
-from .safetensors import SafetensorsReader, bf16_to_f32, f32_to_bf16
+from .hybrid import DTYPES, HybridModel, Packer, load_folder
+from .runtime import BF16
 
 MIXERS = {"attention": 0, "general_delta": 1}  # SKN_MIX_*
-DTYPES = {"bfloat16": BF16, "float32": F32}
 
 
 @dataclass
@@ -99,60 +94,7 @@ def tensor_shapes(cfg: Config, rank: int) -> dict:
     return s
 
 
-def _pad(n, to):
-    return -(-n // to) * to
-
-
-class _Packer:
-    """Tensors of a source (name -> float32 array or bfloat16 bit patterns) in the layout of skn_hybrid_layer."""
-
-    def __init__(self, source, weight_type):
-        self.get, self.type = source, weight_type
-
-    def matrix(self, name, shape):
-        a = self.get(name)
-        if tuple(a.shape) != tuple(shape):
-            raise ValueError(f"{name} is {tuple(a.shape)}, expected {tuple(shape)}")
-        if self.type == F32:
-            return bf16_to_f32(a) if a.dtype == np.uint16 else np.asarray(a, dtype=np.float32)
-        return a if a.dtype == np.uint16 else f32_to_bf16(a)
-
-    def vector(self, name, n):
-        a = self.get(name)
-        if tuple(a.shape) != (n,):
-            raise ValueError(f"{name} is {tuple(a.shape)}, expected {(n,)}")
-        return bf16_to_f32(a) if a.dtype == np.uint16 else np.asarray(a, dtype=np.float32)
-
-    def zeros(self, rows, cols):
-        return np.zeros((rows, cols), dtype=np.float32 if self.type == F32 else np.uint16)
-
-    def stack(self, parts, k):
-        """[(name, rows)] one below the other, each from a multiple of 32 rows, columns padded to a multiple of 64."""
-        out, at = self.zeros(sum(_pad(r, 32) for _, r in parts), _pad(k, 64)), 0
-        for name, rows in parts:
-            out[at:at + rows, :k] = self.matrix(name, (rows, k))
-            at += _pad(rows, 32)
-        return out
-
-    def beside(self, parts, rows):
-        """[(name, columns)] side by side, each from a multiple of 64 columns, rows padded to a multiple of 32."""
-        out, at = self.zeros(_pad(rows, 32), sum(_pad(k, 64) for _, k in parts)), 0
-        for name, k in parts:
-            out[:rows, at:at + k] = self.matrix(name, (rows, k))
-            at += _pad(k, 64)
-        return out
-
-    def padded(self, parts, to):
-        """[(name or None, n)] vectors one after the other, each padded to a multiple of `to` (None: zeros)."""
-        out, at = np.zeros(sum(_pad(n, to) for _, n in parts), dtype=np.float32), 0
-        for name, n in parts:
-            if name is not None:
-                out[at:at + n] = self.vector(name, n)
-            at += _pad(n, to)
-        return out
-
-
-def _pack_layer(pk: _Packer, cfg: Config, i: int):
+def _pack_layer(pk: Packer, cfg: Config, i: int):
     """-> (scalars of the layer's struct, its arrays by field name)"""
     layer, p, w = cfg.layers[i], f"l{i}.mix.", cfg.width
     c, g = layer.columns, layer.kv_heads * layer.dim
@@ -181,58 +123,16 @@ def _pack_layer(pk: _Packer, cfg: Config, i: int):
     return scalars, arrays
 
 
-class NusilixModel(DecoderModel):
-    """Device-resident model: owns the uploaded weights and the skn_hybrid handle."""
+class NusilixModel(HybridModel):
+    def pack_layer(self, pk, i):
+        return _pack_layer(pk, self.cfg, i)
 
-    PREFIX = "skn_hybrid"
-
-    def __init__(self, ctx: runtime.Context, cfg: Config, source):
-        """source(name) -> float32 array or bfloat16 bit patterns (uint16)."""
-        self.ctx, self.cfg, self.bufs = ctx, cfg, {}
-        pk = _Packer(source, cfg.weight_type)
-        self.weight_bytes = 0  # of the matrices a decode step streams
-        layers = (HybridLayer * cfg.n_layer)()
-        for i in range(cfg.n_layer):
-            scalars, arrays = _pack_layer(pk, cfg, i)
-            for k, v in scalars.items():
-                setattr(layers[i], k, v)
-            for k, a in arrays.items():
-                self.bufs[f"l{i}.{k}"] = ctx.to_device(a)
-                setattr(layers[i], k, self.bufs[f"l{i}.{k}"].ptr)
-                if k in ("w_in", "w_out", "w_decay"):
-                    self.weight_bytes += a.nbytes
-        for name, a in (("embed", pk.stack([("embed", cfg.vocab)], cfg.width)), ("final_norm", pk.padded([("final.norm", cfg.width)], 64)),
-                        ("head", pk.stack([("head", cfg.vocab)], cfg.width))):
-            self.bufs[name] = ctx.to_device(a)
-            if name == "head":
-                self.weight_bytes += a.nbytes
-        w = HybridWeights(self.bufs["embed"].ptr, self.bufs["final_norm"].ptr, self.bufs["head"].ptr, layers)
-        c = HybridConfig(cfg.n_layer, cfg.width, cfg.vocab, cfg.max_tokens, cfg.page_tokens, cfg.norm_groups, cfg.weight_type, cfg.norm_eps,
-                         cfg.residual_mult)
-        h = C.c_void_p()
-        ctx._check(ctx.lib.skn_hybrid_create(ctx.handle, C.byref(c), C.byref(w), C.byref(h)))
-        self.handle = h.value
-
-    def extend(self, tokens, want=()):
-        """The next tokens of the sequence as given; -> logits after the tokens at the places `want` (any order), [len(want), vocab]."""
-        toks = np.ascontiguousarray(tokens, dtype=np.int32)
-        want = np.asarray(list(want), dtype=np.int32)
-        order = np.argsort(want, kind="stable")
-        rows = np.ascontiguousarray(want[order])
-        out = np.empty((len(rows), self.cfg.vocab), dtype=np.float32)
-        i32 = C.POINTER(C.c_int32)
-        self._call("extend", toks.ctypes.data_as(i32), len(toks), rows.ctypes.data_as(i32), len(rows), out.ctypes.data)
-        res = np.empty_like(out)
-        res[order] = out
-        return res
+    def pack_model(self, pk):
+        cfg = self.cfg
+        return {"norm_groups": cfg.norm_groups, "residual_mult": cfg.residual_mult, "sinusoid": 1}, {
+            "embed": pk.stack([("embed", cfg.vocab)], cfg.width), "final_norm": pk.padded([("final.norm", cfg.width)], 64),
+            "head": pk.stack([("head", cfg.vocab)], cfg.width)}
 
 
 def load(ctx: runtime.Context, path: str, dtype="bfloat16", max_tokens=None, page_tokens=256) -> NusilixModel:
-    """A folder with config.json and model.safetensors."""
-    with open(os.path.join(path, "config.json")) as f:
-        cfg = config_from_json(json.load(f), max_tokens or 2048, page_tokens, dtype)
-    reader = SafetensorsReader(os.path.join(path, "model.safetensors"))
-    try:
-        return NusilixModel(ctx, cfg, lambda name: reader.raw(name) if reader.dtype(name) == "BF16" else reader.f32(name))
-    finally:
-        reader.close()
+    return load_folder(ctx, path, config_from_json, NusilixModel, dtype, max_tokens, page_tokens)

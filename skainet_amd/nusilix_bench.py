@@ -7,6 +7,7 @@ import time
 import numpy as np
 
 from . import llama, nusilix
+from .safetensors import f32_to_bf16
 
 HBM_PEAK = 8.0e12
 BF16_PEAK = 2.5e15
@@ -42,7 +43,7 @@ def random_source(cfg, rank, seed=7):
             v = 1.0 + 0.1 * rng.standard_normal(shape) if "norm" in name else 0.1 * rng.standard_normal(shape)
             return v.astype(np.float32)
         if shape[1] not in scaled:
-            scaled[shape[1]] = nusilix.f32_to_bf16(block / np.sqrt(shape[1]))
+            scaled[shape[1]] = f32_to_bf16(block / np.sqrt(shape[1]))
         b = np.roll(scaled[shape[1]], int(rng.integers(1 << 22)))
         return np.resize(b, shape)
 

@@ -64,10 +64,33 @@ class SharedAttn(C.Structure):
     ]
 
 
+class RangedAttn(C.Structure):
+    _fields_ = [
+        ("n_head", C.c_int32), ("mask", C.c_int32), ("mask_size", C.c_int32), ("sink", C.c_int32), ("rot_dims", C.c_int32), ("scale", C.c_float),
+        ("softcap", C.c_float), ("eps", C.c_float), ("q_norm", C.c_void_p), ("k_norm", C.c_void_p), ("rot_freq", C.c_void_p),
+    ]
+
+
+class LatentAttn(C.Structure):
+    _fields_ = [
+        ("n_head", C.c_int32), ("dim", C.c_int32), ("rot_dim", C.c_int32), ("vdim", C.c_int32), ("rank", C.c_int32), ("mask", C.c_int32),
+        ("mask_size", C.c_int32), ("scale", C.c_float), ("eps", C.c_float), ("norm", C.c_void_p), ("rot_freq", C.c_void_p), ("w_up", C.c_void_p),
+        ("w_type", C.c_int32),
+    ]
+
+
+class ChannelDelta(C.Structure):
+    _fields_ = [("conv", C.c_void_p), ("decay_rate", C.c_void_p)]
+
+
+MASKS = {None: 0, "window": 1, "chunk": 2}  # SKN_MASK_*
+
+
 class HybridConfig(C.Structure):
     _fields_ = [
         ("n_layer", C.c_int32), ("width", C.c_int32), ("vocab", C.c_int32), ("max_tokens", C.c_int32), ("page_tokens", C.c_int32),
         ("norm_groups", C.c_int32), ("weight_type", C.c_int32), ("norm_eps", C.c_float), ("residual_mult", C.c_float),
+        ("embed_scale", C.c_float), ("sinusoid", C.c_int32), ("side_dim", C.c_int32),
     ]
 
 
@@ -77,11 +100,16 @@ class HybridLayer(C.Structure):
         ("scale", C.c_float), ("temp_coef", C.c_float), ("temp_every", C.c_float), ("act_pos", C.c_float), ("act_neg", C.c_float),
         ("norm", C.c_void_p), ("w_in", C.c_void_p), ("b_in", C.c_void_p), ("w_out", C.c_void_p), ("b_out", C.c_void_p),
         ("q_norm", C.c_void_p), ("k_norm", C.c_void_p), ("w_decay", C.c_void_p), ("b_decay", C.c_void_p), ("o_norm", C.c_void_p),
+        ("vdim", C.c_int32), ("mask", C.c_int32), ("mask_size", C.c_int32), ("sink", C.c_int32), ("rot_dims", C.c_int32), ("kv_rank", C.c_int32),
+        ("kv_from", C.c_int32), ("taps", C.c_int32), ("rank_gate", C.c_int32), ("act", C.c_int32), ("softcap", C.c_float), ("rot_base", C.c_double),
+        ("norm2", C.c_void_p), ("w_up", C.c_void_p), ("w_down", C.c_void_p), ("w_latent", C.c_void_p), ("latent_norm", C.c_void_p),
+        ("w_gate", C.c_void_p), ("conv", C.c_void_p), ("decay_rate", C.c_void_p), ("side_gate", C.c_void_p), ("side_proj", C.c_void_p),
+        ("side_norm", C.c_void_p),
     ]
 
 
 class HybridWeights(C.Structure):
-    _fields_ = [("embed", C.c_void_p), ("final_norm", C.c_void_p), ("head", C.c_void_p), ("layers", C.POINTER(HybridLayer))]
+    _fields_ = [("embed", C.c_void_p), ("final_norm", C.c_void_p), ("head", C.c_void_p), ("layers", C.POINTER(HybridLayer)), ("side", C.c_void_p)]
 
 
 _SIGNATURES = {
@@ -134,12 +162,19 @@ _SIGNATURES = {
     "skn_attn_prefill": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_float, C.c_void_p]),
     "skn_kv_create_shared": (C.c_int, [C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.POINTER(C.c_void_p)]),
     "skn_attn_shared": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int, C.POINTER(SharedAttn), C.c_void_p, C.c_void_p, C.c_int, C.c_void_p]),
+    "skn_kv_create_ranged": (C.c_int, [C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.POINTER(C.c_void_p)]),
+    "skn_attn_ranged": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int, C.POINTER(RangedAttn), C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p]),
+    "skn_kv_create_latent": (C.c_int, [C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.POINTER(C.c_void_p)]),
+    "skn_attn_latent": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int, C.POINTER(LatentAttn), C.c_void_p, C.c_void_p, C.c_int, C.c_void_p]),
+    "skn_rstate_create_conv": (C.c_int, [C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.POINTER(C.c_void_p)]),
+    "skn_gated_delta": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int, C.POINTER(ChannelDelta), C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p]),
     "skn_rstate_create": (C.c_int, [C.c_void_p, C.c_int, C.c_int, C.c_int, C.POINTER(C.c_void_p)]),
     "skn_rstate_free": (C.c_int, [C.c_void_p, C.c_void_p]),
     "skn_rstate_reset": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int]),
     "skn_delta_rule": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p]),
     "skn_rmsnorm_grouped": (C.c_int, [C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_float, C.c_void_p]),
     "skn_xielu": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int64, C.c_float, C.c_float, C.c_void_p]),
+    "skn_gelu": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int64, C.c_void_p]),
     "skn_rmsnorm": (C.c_int, [C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_int, C.c_float, C.c_void_p]),
     "skn_rope": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_int, C.c_float]),
     "skn_swiglu": (C.c_int, [C.c_void_p, C.c_void_p, C.c_void_p, C.c_int64, C.c_void_p]),
@@ -406,6 +441,91 @@ class RecurrentState:
             self.handle = None
 
 
+def _upload(ctx, array, dtype=np.float32):
+    return None if array is None else ctx.to_device(np.ascontiguousarray(array, dtype=dtype))
+
+
+def _rot_freq(base, dims):
+    return base ** (-2.0 * np.arange(dims // 2) / dims) if dims else np.ones(1)
+
+
+class RangedKVCache:
+    """A cache of keys and values of their own sizes (skn_kv_create_ranged)."""
+
+    def __init__(self, ctx, n_seq, n_head, dim, vdim, page_tokens, max_tokens, elem_type=F16):
+        self.ctx, self.n_head, self.dim, self.vdim = ctx, n_head, dim, vdim
+        h = C.c_void_p()
+        ctx._check(ctx.lib.skn_kv_create_ranged(ctx.handle, n_seq, n_head, dim, vdim, elem_type, page_tokens, max_tokens, C.byref(h)))
+        self.handle = h.value
+
+    def attend(self, seq, params, q, k, v, gate=None):
+        """The next tokens of a sequence: host arrays q [n, heads * dim], k [n, n_head * dim], v [n, n_head * vdim], gate [n, heads * vdim]
+        or None -> [n, heads * vdim].  params: dict with n_head, scale, eps and optionally mask ("window" / "chunk", size),
+        sink, softcap, rot_dims, rot_base, q_norm, k_norm."""
+        ctx, g = self.ctx, params.get
+        keep = [_upload(ctx, a) for a in (q, k, v, gate, g("q_norm"), g("k_norm"))]
+        freq = _upload(ctx, _rot_freq(g("rot_base", 10000.0), g("rot_dims", 0)), np.float64)
+        mask, size = g("mask") or (None, 0)
+        p = RangedAttn(params["n_head"], MASKS[mask], size, int(g("sink", 0)), g("rot_dims", 0), params["scale"], g("softcap", 0.0), params["eps"],
+                       _ptr(keep[4]), _ptr(keep[5]), freq.ptr)
+        n, cols = len(q), params["n_head"] * self.vdim
+        out = ctx.alloc(n * cols * 4)
+        ctx._check(ctx.lib.skn_attn_ranged(ctx.handle, self.handle, seq, C.byref(p), *(_ptr(b) for b in keep[:4]), n, out.ptr))
+        return out.download(np.float32, n * cols).reshape(n, cols)
+
+    reset, length, free = SharedKVCache.reset, SharedKVCache.length, SharedKVCache.free
+
+
+class LatentKVCache:
+    """A cache of latents with rotated key parts (skn_kv_create_latent)."""
+
+    def __init__(self, ctx, n_seq, rank, rot_dim, page_tokens, max_tokens, elem_type=F16):
+        self.ctx, self.rank, self.rot_dim = ctx, rank, rot_dim
+        h = C.c_void_p()
+        ctx._check(ctx.lib.skn_kv_create_latent(ctx.handle, n_seq, rank, rot_dim, elem_type, page_tokens, max_tokens, C.byref(h)))
+        self.handle = h.value
+
+    def attend(self, seq, params, q, d=None):
+        """The next tokens of a sequence: host arrays q [n, heads * (dim + rot_dim)], d [n, rank + rot_dim] -> [n, heads * vdim]; without
+        d the last tokens of the cache again.  params: dict with n_head, dim, vdim, scale, eps, norm, w_up (as laid out by
+        skn_latent_attn, float32 or bfloat16 bit patterns), and optionally mask and rot_base."""
+        ctx, g = self.ctx, params.get
+        w = params["w_up"]
+        keep = [_upload(ctx, a) for a in (q, d, g("norm"))] + [_upload(ctx, w, w.dtype)]
+        freq = _upload(ctx, _rot_freq(g("rot_base", 10000.0), self.rot_dim), np.float64)
+        mask, size = g("mask") or (None, 0)
+        p = LatentAttn(params["n_head"], params["dim"], self.rot_dim, params["vdim"], self.rank, MASKS[mask], size, params["scale"], params["eps"],
+                       _ptr(keep[2]), freq.ptr, keep[3].ptr, BF16 if w.dtype == np.uint16 else F32)
+        n, cols = len(q), params["n_head"] * params["vdim"]
+        out = ctx.alloc(n * cols * 4)
+        ctx._check(ctx.lib.skn_attn_latent(ctx.handle, self.handle, seq, C.byref(p), _ptr(keep[0]), _ptr(keep[1]), n, out.ptr))
+        return out.download(np.float32, n * cols).reshape(n, cols)
+
+    reset, length, free = SharedKVCache.reset, SharedKVCache.length, SharedKVCache.free
+
+
+class ConvRecurrentState:
+    """State of gated delta rule layers behind short convolutions (skn_rstate_create_conv)."""
+
+    def __init__(self, ctx, n_seq, heads, kv_heads, dim, vdim, taps):
+        self.ctx, self.heads, self.vdim = ctx, heads, vdim
+        h = C.c_void_p()
+        ctx._check(ctx.lib.skn_rstate_create_conv(ctx.handle, n_seq, heads, kv_heads, dim, vdim, taps, C.byref(h)))
+        self.handle = h.value
+
+    def advance(self, seq, conv, decay_rate, q, k, v, beta, z):
+        """The next tokens of a sequence: host arrays as skn_gated_delta takes them -> outputs [n, heads * vdim]."""
+        ctx = self.ctx
+        keep = [_upload(ctx, a) for a in (conv, decay_rate, q, k, v, beta, z)]
+        p = ChannelDelta(keep[0].ptr, keep[1].ptr)
+        n, cols = len(q), self.heads * self.vdim
+        out = ctx.alloc(n * cols * 4)
+        ctx._check(ctx.lib.skn_gated_delta(ctx.handle, self.handle, seq, C.byref(p), *(b.ptr for b in keep[2:]), n, out.ptr))
+        return out.download(np.float32, n * cols).reshape(n, cols)
+
+    reset, free = RecurrentState.reset, RecurrentState.free
+
+
 def _ptr(x):
     if isinstance(x, DeviceBuffer):
         return x.ptr
@@ -536,6 +656,9 @@ class Context:
 
     def xielu(self, z_dev, n, pos, neg, out_dev):
         self._check(self.lib.skn_xielu(self.handle, _ptr(z_dev), n, pos, neg, _ptr(out_dev)))
+
+    def gelu(self, z_dev, n, out_dev):
+        self._check(self.lib.skn_gelu(self.handle, _ptr(z_dev), n, _ptr(out_dev)))
 
     def rope(self, x_dev, rows, n_head, head_dim, pos0, base):
         self._check(self.lib.skn_rope(self.handle, _ptr(x_dev), rows, n_head, head_dim, pos0, base))

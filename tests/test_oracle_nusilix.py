@@ -7,7 +7,7 @@ import numpy as np
 import pytest
 
 from oracle import nusilix_oracle as orc
-from skainet_amd import models, nusilix
+from skainet_amd import hybrid, models, nusilix
 from skainet_amd.safetensors import SafetensorsReader, bf16_to_f32, f32_to_bf16, write_safetensors
 
 
@@ -143,7 +143,7 @@ def test_packed_layer_holds_every_weight_once():
     """The stacked and joined matrices of a layer multiply like the separate ones."""
     cfg_dict, rank = cases.MODELS["mixed"]
     cfg, w = nusilix.config_from_json(cfg_dict, dtype="float32"), cases.weights(cfg_dict, rank)
-    pk = nusilix._Packer(lambda n: w[n], cfg.weight_type)
+    pk = hybrid.Packer(lambda n: w[n], cfg.weight_type)
     x = np.random.default_rng(0).standard_normal(cfg.width).astype(np.float32)
     xp = np.zeros(192, dtype=np.float32)
     xp[:cfg.width] = x
@@ -167,7 +167,7 @@ def test_missing_or_misshapen_tensors_are_named():
     cfg, w = nusilix.config_from_json(cfg_dict), cases.weights(cfg_dict, rank)
     w["l1.mix.q"] = w["l1.mix.q"][:-1]
     with pytest.raises(ValueError, match="l1.mix.q"):
-        nusilix._pack_layer(nusilix._Packer(lambda n: w[n], cfg.weight_type), cfg, 1)
+        nusilix._pack_layer(hybrid.Packer(lambda n: w[n], cfg.weight_type), cfg, 1)
 
 
 def test_registry(tmp_path):
