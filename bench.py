@@ -404,8 +404,8 @@ def main():
     ap.add_argument("--warmup", type=int, default=100)
     ap.add_argument("--no-cpu", action="store_true", help="skip the CPU baseline leg")
     ap.add_argument("--no-extra", action="store_true", help="skip the secondary shapes")
-    ap.add_argument("--mode", choices=["bench", "copy", "decode", "attention", "gemm", "formats", "timeline", "ksplit", "nusilix"], default="bench",
-                    help="decode / attention / gemm: only that leg (for kernel traces).  nusilix: prefill and decode of Nusilix models beside the Llama-style decoder of equal size.  timeline: the headline kernel's in-kernel time stamps.  ksplit: the headline matvec with k split across workgroups beside the default.  copy: run --steps plain device copies of the headline weight size instead (the known-size "
+    ap.add_argument("--mode", choices=["bench", "copy", "decode", "attention", "gemm", "formats", "timeline", "ksplit", "nusilix", "lebelix"], default="bench",
+                    help="decode / attention / gemm: only that leg (for kernel traces).  nusilix: prefill and decode of Nusilix models beside the Llama-style decoder of equal size.  lebelix: of Lebelix models beside the Nusilix decoder of equal size.  timeline: the headline kernel's in-kernel time stamps.  ksplit: the headline matvec with k split across workgroups beside the default.  copy: run --steps plain device copies of the headline weight size instead (the known-size "
                          "workload that hardware traffic counters are calibrated against)")
     ap.add_argument("--set", action="append", default=[], metavar="KEY=VALUE",
                     help="a tuning option of the library (skn_set_option) for this run, e.g. --set attn.splits=2 or --set llama.attn_wide=0; repeatable")
@@ -413,7 +413,9 @@ def main():
                     help="decode without the captured step graph (kernel tracers that cannot follow graph launches)")
     ap.add_argument("--nusilix", default="2048:both,4096:both", metavar="SIZE:KIND,...",
                     help="--mode nusilix: widths (2048, 4096) and layer kinds (both, attention, general_delta; llama: the other decoder alone) to run")
-    ap.add_argument("--no-beside", action="store_true", help="--mode nusilix: without the Llama-style decoder")
+    ap.add_argument("--lebelix", default="2048:all,4096:all", metavar="SIZE:KIND,...",
+                    help="--mode lebelix: widths (2048, 4096) and layer kinds (all, attention, latent_attention, channel_delta; nusilix or nusilix-KIND: the other decoder alone) to run")
+    ap.add_argument("--no-beside", action="store_true", help="--mode nusilix, lebelix: without the other decoder")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build runs on one GPU only (no collectives, no sharding); use --gpus 1", file=sys.stderr)
@@ -448,13 +450,13 @@ def main():
                           "read_plus_write_gbs": round(2 * nbytes / (ms / launches * 1e-3) / 1e9, 1)}))
         ctx.close()
         return
-    if args.mode == "nusilix":
-        from skainet_amd import nusilix_bench
-        rows = {}
-        for item in args.nusilix.split(","):
+    if args.mode in ("nusilix", "lebelix"):
+        from skainet_amd import lebelix_bench, nusilix_bench
+        rows, items, runner = {}, {"nusilix": args.nusilix, "lebelix": args.lebelix}[args.mode], {"nusilix": nusilix_bench, "lebelix": lebelix_bench}[args.mode]
+        for item in items.split(","):
             size, _, kinds = item.partition(":")
-            rows[item] = nusilix_bench.run(ctx, size, kinds or "both", steps=min(args.steps, 64), beside=not args.no_beside)
-        print(json.dumps({"mode": "nusilix", "data": "synthetic, random weights", "dtype": "bf16", **rows}))
+            rows[item] = runner.run(ctx, size, *([kinds] if kinds else []), steps=min(args.steps, 64), beside=not args.no_beside)
+        print(json.dumps({"mode": args.mode, "data": "synthetic, random weights", "dtype": "bf16", **rows}))
         ctx.close()
         return
     if args.mode == "decode":

@@ -79,6 +79,11 @@ def sink_softmax(s, mask):
     return e / (np.exp(-m) + e.sum(axis=-1, keepdims=True))
 
 
+def heads_first(x):
+    """[T, H, D] to [H, T, D], and back"""
+    return np.swapaxes(x, 0, 1)
+
+
 def causal_conv(x, taps):
     """x [T, C], taps [C, K]: the last column of taps meets the token itself, zeros lie before the start."""
     K = taps.shape[1]
@@ -133,9 +138,9 @@ def latent_attention_mixer(h, w, pre, m, eps, shared=None):
     c, k_rot = shared if shared is not None else latent_row(h, w, pre, m, eps)
     k = (c @ w[pre + "uk"].T).reshape(T, H, D)
     v = (c @ w[pre + "uv"].T).reshape(T, H, V)
-    s = (np.einsum("thd,shd->hts", q[..., :D], k) + np.einsum("thd,sd->hts", q_rot, k_rot)) * m["scale"]
+    s = (heads_first(q[..., :D]) @ heads_first(k).swapaxes(1, 2) + heads_first(q_rot) @ k_rot.T) * m["scale"]
     p = softmax(s, window_mask(T, m["mask"]["size"]))
-    return np.einsum("hts,shv->thv", p, v).reshape(T, H * V) @ w[pre + "o"].T
+    return heads_first(p @ heads_first(v)).reshape(T, H * V) @ w[pre + "o"].T
 
 
 def attention_mixer(h, w, pre, m, eps, shared=None):
@@ -145,9 +150,9 @@ def attention_mixer(h, w, pre, m, eps, shared=None):
     k = plain_norm(k.reshape(T, G, D), w[pre + "k.norm"], eps)
     q, k = (rotate_half(x, np.arange(T), m["rot"]["base"], m["rot"]["dims"]) for x in (q, k))
     of_head = np.arange(H) // (H // G)
-    s = soft_cap(np.einsum("thd,shd->hts", q, k[:, of_head]) * m["scale"], m["softcap"])
+    s = soft_cap(heads_first(q) @ heads_first(k[:, of_head]).swapaxes(1, 2) * m["scale"], m["softcap"])
     p = sink_softmax(s, chunk_mask(T, m["mask"]["size"]))
-    o = np.einsum("hts,shv->thv", p, v.reshape(T, G, V)[:, of_head]).reshape(T, H * V)
+    o = heads_first(p @ heads_first(v.reshape(T, G, V)[:, of_head])).reshape(T, H * V)
     return (o * sigmoid(h @ w[pre + "g"].T)) @ w[pre + "o"].T
 
 

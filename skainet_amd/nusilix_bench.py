@@ -30,9 +30,8 @@ def config(size, kinds="both", max_tokens=8192):
                           max_tokens=max_tokens)
 
 
-def random_source(cfg, rank, seed=7):
-    """source(name) for nusilix.NusilixModel: bfloat16 patterns cut out of one random block, matrices scaled by 1 / sqrt(columns)."""
-    shapes = nusilix.tensor_shapes(cfg, rank)
+def random_source(shapes, seed=7):
+    """source(name) of a model with these tensors: bfloat16 patterns cut out of one random block, matrices scaled by 1 / sqrt(columns)."""
     rng = np.random.default_rng(seed)
     block = rng.standard_normal(1 << 22).astype(np.float32)
     scaled = {}
@@ -73,7 +72,7 @@ def prompt_flops(cfg, rank, n):
     return total
 
 
-def _timed(ctx, fn, reps):
+def timed(ctx, fn, reps):
     fn()
     ctx.sync()
     best = 1e9
@@ -85,7 +84,7 @@ def _timed(ctx, fn, reps):
     return best
 
 
-def _measure(ctx, model, prompts, contexts, steps, rng, vocab):
+def measure(ctx, model, prompts, contexts, steps, rng, vocab):
     out = {}
     for n in prompts:
         prompt = rng.integers(0, vocab, n).tolist()
@@ -94,7 +93,7 @@ def _measure(ctx, model, prompts, contexts, steps, rng, vocab):
             model.reset()
             model.prefill(prompt)
 
-        out[f"prefill_{n}"] = _timed(ctx, prefill, 3)
+        out[f"prefill_{n}"] = timed(ctx, prefill, 3)
     for n in contexts:
         model.reset()
         first = model.prefill(rng.integers(0, vocab, n).tolist())
@@ -113,10 +112,10 @@ def run(ctx, size, kinds="both", prompts=(512, 2048), contexts=(512, 4096), step
         return run_llama(ctx, size, prompts, contexts, steps)
     _, _, _, _, _, _, _, rank, n_layer = SIZES[size]
     cfg = config(size, kinds)
-    model = nusilix.NusilixModel(ctx, cfg, random_source(cfg, rank))
-    t = _measure(ctx, model, prompts, contexts, steps, np.random.default_rng(3), VOCAB)
+    model = nusilix.NusilixModel(ctx, cfg, random_source(nusilix.tensor_shapes(cfg, rank)))
+    t = measure(ctx, model, prompts, contexts, steps, np.random.default_rng(3), VOCAB)
     out = {"layers": f"{n_layer} x {kinds}", "weight_mb": round(model.weight_bytes / 1e6, 1)}
-    _report(out, t, {n: prompt_flops(cfg, rank, n) for n in prompts}, {n: decode_bytes(cfg, model, n + steps / 2) for n in contexts})
+    report(out, t, {n: prompt_flops(cfg, rank, n) for n in prompts}, {n: decode_bytes(cfg, model, n + steps / 2) for n in contexts})
     model.free()
     if beside:
         out["llama_q4_k_beside"] = run_llama(ctx, size, prompts, contexts, steps)
@@ -128,17 +127,17 @@ def run_llama(ctx, size, prompts, contexts, steps):
     w, ff, h, kv, d, _, _, _, n_layer = SIZES[size]
     cfg = llama.Config(n_layer=n_layer, hidden=w, ffn=ff, n_head=h, head_dim=d, vocab=VOCAB, max_tokens=8192, n_kv_head=kv)
     model = llama.LlamaModel(ctx, cfg, seed=5)
-    t = _measure(ctx, model, prompts, contexts, steps, np.random.default_rng(3), VOCAB)
+    t = measure(ctx, model, prompts, contexts, steps, np.random.default_rng(3), VOCAB)
     weights = model.weight_bytes_per_token()
     out = {"weight_mb": round(weights / 1e6, 1)}
     params = n_layer * (2 * w * w + 2 * w * kv * d + 3 * w * ff)
-    _report(out, t, {n: 2 * params * n + n_layer * 4 * n * (n + 1) // 2 * w for n in prompts},
+    report(out, t, {n: 2 * params * n + n_layer * 4 * n * (n + 1) // 2 * w for n in prompts},
             {n: weights + n_layer * (n + steps / 2) * 2 * 2 * kv * d for n in contexts})
     model.free()
     return out
 
 
-def _report(out, t, flops, nbytes):
+def report(out, t, flops, nbytes):
     for n, f in flops.items():
         s = t[f"prefill_{n}"]
         out[f"prefill_{n}"] = {"ms": round(s * 1e3, 3), "tok_s": round(n / s, 1), "frac_bf16_peak": round(f / s / BF16_PEAK, 4)}
