@@ -115,7 +115,9 @@ __global__ __launch_bounds__(1024) void latent_prep_kernel(const LatentArgs a) {
     }
 }
 
-// grid (heads, rows), eight wavefronts: the head's latent (merged from the splits) in LDS, then a wavefront per row of Wuv
+constexpr int kValueRows = 32;
+// grid (heads, rows, rows of Wuv / 32), eight wavefronts: the head's latent (merged from the splits) in LDS, then four rows of Wuv per
+// wavefront
 template <typename W>
 __global__ __launch_bounds__(512) void latent_value_kernel(const skn_latent_attn p, int row0, int rank_pad, int width, const float* __restrict__ lat, int splits,
                                                            const float* __restrict__ ml, void* __restrict__ out, int ldo, int out_type) {
@@ -123,19 +125,25 @@ __global__ __launch_bounds__(512) void latent_value_kernel(const skn_latent_attn
     const int h = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, rank = p.rank;
     if (splits > 1) {
         float m = -INFINITY, l = 0.f, f[kMaxSplits];
-        for (int i = 0; i < splits; i++) m = fmaxf(m, ml[2 * (i * p.n_head + h)]);
+        float2 part[kMaxSplits];  // (all requested before the first is used)
+#pragma unroll
+        for (int i = 0; i < kMaxSplits; i++) part[i] = reinterpret_cast<const float2*>(ml)[min(i, splits - 1) * p.n_head + h];
+#pragma unroll
+        for (int i = 0; i < kMaxSplits; i++) m = fmaxf(m, part[i].x);
 #pragma unroll
         for (int i = 0; i < kMaxSplits; i++) {
-            f[i] = i < splits ? __builtin_amdgcn_exp2f(ml[2 * (min(i, splits - 1) * p.n_head + h)] - m) : 0.f;
-            l = fmaf(f[i], ml[2 * (min(i, splits - 1) * p.n_head + h) + 1], l);
+            f[i] = i < splits ? __builtin_amdgcn_exp2f(part[i].x - m) : 0.f;
+            l = fmaf(f[i], part[i].y, l);
         }
         const float inv = 1.0f / l;
         for (int i = tid; i < rank_pad; i += 512) {
             float a = 0.f;
             if (i < rank) {
+                float y[kMaxSplits];
 #pragma unroll
-                for (int s = 0; s < kMaxSplits; s++)
-                    if (s < splits) a = fmaf(f[s], lat[((int64_t)s * p.n_head + h) * width + i], a);
+                for (int s = 0; s < kMaxSplits; s++) y[s] = lat[((int64_t)min(s, splits - 1) * p.n_head + h) * width + i];
+#pragma unroll
+                for (int s = 0; s < kMaxSplits; s++) a = fmaf(f[s], y[s], a);
             }
             x[i] = a * inv;
         }
@@ -144,20 +152,24 @@ __global__ __launch_bounds__(512) void latent_value_kernel(const skn_latent_attn
     }
     __syncthreads();
     const W* w = (const W*)p.w_up + ((int64_t)row0 + h * p.vdim) * rank_pad;
-    for (int v = wave; v < p.vdim; v += 8) {
-        float s = 0.f;
-        for (int pc = lane; pc < rank_pad >> 3; pc += 64) {
-            float f[8];
-            load_weights8(w + (int64_t)v * rank_pad + 8 * pc, f);
-            const float4 a = reinterpret_cast<const float4*>(x)[2 * pc], b = reinterpret_cast<const float4*>(x)[2 * pc + 1];
-            s += ((f[0] * a.x + f[1] * a.y) + (f[2] * a.z + f[3] * a.w)) + ((f[4] * b.x + f[5] * b.y) + (f[6] * b.z + f[7] * b.w));
-        }
-        s = wave_sum(s);
-        if (lane == 0) {
-            const int64_t at = (int64_t)row * ldo + h * p.vdim + v;
-            if (out_type == SKN_TYPE_F32) ((float*)out)[at] = s;
-            else ((uint16_t*)out)[at] = skn_bf16_bits(s);
-        }
+    const int v0 = blockIdx.z * kValueRows + wave * 4;
+    float s[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int pc = lane; pc < rank_pad >> 3; pc += 64) {
+        float f[4][8];
+#pragma unroll
+        for (int r = 0; r < 4; r++) load_weights8(w + (int64_t)min(v0 + r, p.vdim - 1) * rank_pad + 8 * pc, f[r]);
+        const float4 a = reinterpret_cast<const float4*>(x)[2 * pc], b = reinterpret_cast<const float4*>(x)[2 * pc + 1];
+#pragma unroll
+        for (int r = 0; r < 4; r++)
+            s[r] += ((f[r][0] * a.x + f[r][1] * a.y) + (f[r][2] * a.z + f[r][3] * a.w)) + ((f[r][4] * b.x + f[r][5] * b.y) + (f[r][6] * b.z + f[r][7] * b.w));
+    }
+#pragma unroll
+    for (int r = 0; r < 4; r++) {
+        s[r] = wave_sum(s[r]);
+        if (lane != 0 || v0 + r >= p.vdim) continue;
+        const int64_t at = (int64_t)row * ldo + h * p.vdim + v0 + r;
+        if (out_type == SKN_TYPE_F32) ((float*)out)[at] = s[r];
+        else ((uint16_t*)out)[at] = skn_bf16_bits(s[r]);
     }
 }
 
@@ -263,7 +275,7 @@ int stream(skn_ctx* ctx, const skn_kv* kv, const StreamArgs& a, int rows) {
 
 int value(skn_ctx* ctx, const skn_kv* kv, const skn_latent_attn& p, const float* lat, int splits, const float* ml, int rows, void* out, int ldo, int out_type) {
     const int rank_pad = skn_pad_cols(p.rank), row0 = skn_pad_rows(p.n_head * p.dim);  // (of Wuv)
-    const dim3 grid(p.n_head, rows);
+    const dim3 grid(p.n_head, rows, (p.vdim + kValueRows - 1) / kValueRows);
     const size_t lds = (size_t)rank_pad * sizeof(float);
     if (p.w_type == SKN_TYPE_F32) skn_launch(ctx, latent_value_kernel<float>, grid, dim3(512), lds, p, row0, rank_pad, kv->head_dim, lat, splits, ml, out, ldo, out_type);
     else skn_launch(ctx, latent_value_kernel<uint16_t>, grid, dim3(512), lds, p, row0, rank_pad, kv->head_dim, lat, splits, ml, out, ldo, out_type);

@@ -25,14 +25,15 @@ typedef float float16_t __attribute__((ext_vector_type(16)));
 
 constexpr int kSlice = 128;  // bytes of k per slice
 
-template <int WM_, int WN_, int TM_, int TN_, int ST_>
+// KG groups of WM x WN wavefronts share the slices of a tile in turn; their sums meet in the epilogue.
+template <int WM_, int WN_, int TM_, int TN_, int ST_, int KG_ = 1>
 struct Shape {
-    static constexpr int WM = WM_, WN = WN_, TM = TM_, TN = TN_, ST = ST_;
-    static constexpr int kThreads = 64 * WM * WN, kRowsA = 32 * TM * WM, kRowsW = 32 * TN * WN;
+    static constexpr int WM = WM_, WN = WN_, TM = TM_, TN = TN_, ST = ST_, KG = KG_;
+    static constexpr int kThreads = 64 * WM * WN * KG, kRowsA = 32 * TM * WM, kRowsW = 32 * TN * WN;
     static constexpr int kBuf = (kRowsA + kRowsW) * kSlice;
     // the epilogue passes 32 WM tokens of the tile at a time through LDS
     static constexpr int kPitch = kRowsW + 4, kOutBytes = 32 * WM * kPitch * 4;
-    static constexpr int kLds = ST * kBuf > kOutBytes ? ST * kBuf : kOutBytes;
+    static constexpr int kLds = KG * (ST * kBuf > kOutBytes ? ST * kBuf : kOutBytes);
 };
 
 __device__ __forceinline__ uint32_t half_bits(float f) { return __half_as_ushort(__float2half_rn(f)); }
@@ -56,10 +57,10 @@ __global__ __launch_bounds__(S::kThreads) void dense_gemm_kernel(const uint8_t* 
                                                                  int64_t ldw_b, int rows, int slices, int tiles_m, int tiles,
                                                                  const float* __restrict__ bias, const skn_dense_out out) {
     extern __shared__ __align__(16) uint8_t lds[];
-    constexpr int WM = S::WM, WN = S::WN, TM = S::TM, TN = S::TN, ST = S::ST, kRowsA = S::kRowsA, kRowsW = S::kRowsW;
+    constexpr int WM = S::WM, WN = S::WN, TM = S::TM, TN = S::TN, ST = S::ST, KG = S::KG, kRowsA = S::kRowsA, kRowsW = S::kRowsW;
     constexpr int kReq = (kRowsA + kRowsW) / 8 / (WM * WN);  // requests per wavefront and slice
     const int tid = threadIdx.x, lane = tid & 63;
-    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int all_wave = __builtin_amdgcn_readfirstlane(tid >> 6), group = all_wave / (WM * WN), wave = all_wave % (WM * WN);
     // An XCD (blockIdx % 8) takes consecutive tiles, which run down up to eight token tiles before they move on to the next
     // weight tile: what is resident on an XCD at a time shares both operands in its L2.
     const int per = (tiles + 7) / 8, tile = (int)(blockIdx.x & 7) * per + (int)(blockIdx.x >> 3);
@@ -77,8 +78,10 @@ __global__ __launch_bounds__(S::kThreads) void dense_gemm_kernel(const uint8_t* 
                                      : w + (int64_t)min(n0 + r - kRowsA, rows - 1) * ldw_b) + piece * 16;
         dst[i] = block * 1024;
     }
-    auto request = [&](int slice) __attribute__((always_inline)) {
-        const int buf = slice % ST * S::kBuf;
+    // the group's i-th slice is slice KG i + group of the tile
+    const int own = (slices - group + KG - 1) / KG, turns = (slices + KG - 1) / KG;
+    auto request = [&](int i_own) __attribute__((always_inline)) {
+        const int buf = (group * ST + i_own % ST) * S::kBuf, slice = KG * i_own + group;
 #pragma unroll
         for (int i = 0; i < kReq; i++)
             __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src[i] + (int64_t)slice * kSlice),
@@ -100,14 +103,15 @@ __global__ __launch_bounds__(S::kThreads) void dense_gemm_kernel(const uint8_t* 
 
 #pragma unroll
     for (int s = 0; s < ST - 1; s++)
-        if (s < slices) request(s);
-    for (int s = 0; s < slices; s++) {
-        // requests complete in order: all but the newest slices' have landed
-        if (s + 1 < slices) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(kReq * (ST - 2)) : "memory");
+        if (s < own) request(s);
+    for (int s = 0; s < turns; s++) {
+        // requests complete in order: all but the newest ST - 2 slices' have landed (near the end there are fewer newer ones: all)
+        if (s + ST - 2 < own) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(kReq * (ST - 2)) : "memory");
         else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-        if (s + ST - 1 < slices) request(s + ST - 1);
-        const int buf = s % ST * S::kBuf;
+        if (s + ST - 1 < own) request(s + ST - 1);
+        if (KG > 1 && s >= own) continue;
+        const int buf = (group * ST + s % ST) * S::kBuf;
         u32x4 fa[2][TM], fw[2][TN];
         auto read = [&](int step) __attribute__((always_inline)) {
             const int off = buf + (((2 * step + h) ^ swz) * 16);
@@ -134,6 +138,7 @@ __global__ __launch_bounds__(S::kThreads) void dense_gemm_kernel(const uint8_t* 
     // of a wavefront store whole rows of the tile.
     constexpr int kPitch = S::kPitch, kQuads = kRowsW / 4;
     float* tile_c = reinterpret_cast<float*>(lds);
+    constexpr int kPart = 32 * WM * kPitch;  // floats of a group's pass
     const int q4 = 4 * (tid % kQuads), row = n0 + q4;  // (this thread's four rows are the same in every turn)
     int si = -1;
     for (int q = 0; q < out.nseg; q++)
@@ -149,14 +154,19 @@ __global__ __launch_bounds__(S::kThreads) void dense_gemm_kernel(const uint8_t* 
         for (int i = 0; i < TN; i++)
 #pragma unroll
             for (int g = 0; g < 4; g++)
-                *reinterpret_cast<float4*>(tile_c + (32 * wv_m + r32) * kPitch + wn + 32 * i + 8 * g + 4 * h) =
+                *reinterpret_cast<float4*>(tile_c + group * kPart + (32 * wv_m + r32) * kPitch + wn + 32 * i + 8 * g + 4 * h) =
                     make_float4(acc[i][j][4 * g], acc[i][j][4 * g + 1], acc[i][j][4 * g + 2], acc[i][j][4 * g + 3]);
         __syncthreads();
         if (left <= 0) continue;
         for (int tl = tid / kQuads; tl < 32 * WM; tl += S::kThreads / kQuads) {
             const int t = m0 + (tl >> 5) * 32 * TM + 32 * j + (tl & 31);
             if (t >= m) continue;
-            const float4 c = *reinterpret_cast<const float4*>(tile_c + tl * kPitch + q4);
+            float4 c = *reinterpret_cast<const float4*>(tile_c + tl * kPitch + q4);
+#pragma unroll
+            for (int k = 1; k < KG; k++) {
+                const float4 d = *reinterpret_cast<const float4*>(tile_c + k * kPart + tl * kPitch + q4);
+                c = make_float4(c.x + d.x, c.y + d.y, c.z + d.z, c.w + d.w);
+            }
             float v[4] = {c.x + b.x, c.y + b.y, c.z + b.z, c.w + b.w};
             if (out.nseg == 0) {
                 float* p = out.resid + (int64_t)t * out.ldr + row;
@@ -196,6 +206,7 @@ __global__ __launch_bounds__(S::kThreads) void dense_gemm_kernel(const uint8_t* 
 }
 
 using Tile64x64 = Shape<2, 2, 1, 1, 3>;
+using Tile32x64Split = Shape<1, 2, 1, 1, 3, 4>;  // for few outputs: more and shorter chains of slices
 using Tile128x64 = Shape<2, 2, 2, 1, 3>;
 using Tile128x128 = Shape<2, 2, 2, 2, 2>;
 using Tile256x256 = Shape<4, 2, 2, 4, 2>;
@@ -228,11 +239,13 @@ int pick_gemm(skn_ctx* ctx, const skn_dense_mat& w, const void* a, int lda, int 
         const float time = tiles / round * c.full + (rest == 0 ? 0.f : rest <= ctx->compute_units ? c.alone : c.full);
         if (time < best_time) best = i, best_time = time;
     }
+    if (((m + 31) / 32) * ((w.rows + 63) / 64) <= ctx->compute_units && w.k_pad * (int)sizeof(T) >= 16 * kSlice) best = 4;
     if (ctx->opt_dense_tile > 0) best = ctx->opt_dense_tile - 1;
     switch (best) {
         case 0: return launch_gemm<T, Tile64x64>(ctx, w, a, lda, m, out);
         case 1: return launch_gemm<T, Tile128x64>(ctx, w, a, lda, m, out);
         case 2: return launch_gemm<T, Tile128x128>(ctx, w, a, lda, m, out);
+        case 4: return launch_gemm<T, Tile32x64Split>(ctx, w, a, lda, m, out);
         default: return launch_gemm<T, Tile256x256>(ctx, w, a, lda, m, out);
     }
 }
@@ -246,6 +259,7 @@ int allow_lds(skn_ctx* ctx) {
 template <typename T>
 int allow_all(skn_ctx* ctx) {
     SKN_TRY((allow_lds<T, Tile64x64>(ctx)));
+    SKN_TRY((allow_lds<T, Tile32x64Split>(ctx)));
     SKN_TRY((allow_lds<T, Tile128x64>(ctx)));
     SKN_TRY((allow_lds<T, Tile128x128>(ctx)));
     return allow_lds<T, Tile256x256>(ctx);

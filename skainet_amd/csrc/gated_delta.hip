@@ -42,44 +42,66 @@ struct ConvArgs {
     float *cq, *ck, *cv;
 };
 
-// channel c (of the ring and the taps) of row t, whose inputs in the portion are src[row * ld]
-__device__ __forceinline__ float conv_row(const ConvArgs& a, const float* src, int c, int t) {
-    float s = 0.f;
-    for (int j = 0; j < a.n_taps; j++) {
-        const int p = a.pos0 + t - j;
-        const float x = j <= t ? src[(int64_t)(t - j) * a.ld] : p >= 0 ? a.ring[(int64_t)(p % a.n_taps) * a.channels + c] : 0.f;
-        s = fmaf(x, a.taps[(int64_t)c * a.n_taps + a.n_taps - 1 - j], s);
+constexpr int kMaxTaps = 8, kConvRows = 8;
+
+// rows t0 .. t0 + 7 of channel c (of the ring and the taps), whose inputs in the portion are src[row * ld]; past the end: the last row
+__device__ __forceinline__ void conv_rows(const ConvArgs& a, const float* src, int c, int t0, float (&y)[kConvRows]) {
+    float w[kMaxTaps], x[kConvRows + kMaxTaps - 1];  // w[j]: of the input j tokens back; x[i]: of row t0 - 7 + i
+#pragma unroll
+    for (int j = 0; j < kMaxTaps; j++) w[j] = j < a.n_taps ? a.taps[(int64_t)c * a.n_taps + a.n_taps - 1 - j] : 0.f;
+#pragma unroll
+    for (int i = 0; i < kConvRows + kMaxTaps - 1; i++) {
+        const int t = t0 - (kMaxTaps - 1) + i, p = a.pos0 + t;
+        x[i] = 0.f;
+        if (i >= kMaxTaps - a.n_taps) {
+            if (t >= 0) x[i] = src[(int64_t)min(t, a.n - 1) * a.ld];
+            else if (p >= 0) x[i] = a.ring[(int64_t)(p % a.n_taps) * a.channels + c];
+        }
     }
-    return silu(s);
+#pragma unroll
+    for (int r = 0; r < kConvRows; r++) {
+        float s = 0.f;
+#pragma unroll
+        for (int j = 0; j < kMaxTaps; j++) s = fmaf(x[r + kMaxTaps - 1 - j], w[j], s);
+        y[r] = silu(s);
+    }
 }
 
-// grid (rows, units / 4): a wavefront takes a q/k head, or 256 value channels
+// grid (rows / 8, units / 4): a wavefront takes the q or the k of a q/k head, or 64 value channels
 __global__ __launch_bounds__(256) void conv_rows_kernel(const ConvArgs a) {
-    const int t = blockIdx.x, unit = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63, qk = a.kv_heads * a.dim;
-    if (unit < a.kv_heads) {
+    const int t0 = blockIdx.x * kConvRows, unit = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63, qk = a.kv_heads * a.dim;
+    const int rows = min(kConvRows, a.n - t0);
+    float y[4][kConvRows];
+    if (unit < 2 * a.kv_heads) {
+        const int which = unit & 1, head = unit >> 1;
+        const float* src = (which ? a.k : a.q) + head * a.dim;
+        float* dst = (which ? a.ck : a.cq) + (int64_t)t0 * a.ld + head * a.dim;
+        float ss[kConvRows];
 #pragma unroll
-        for (int which = 0; which < 2; which++) {
-            const float* src = (which ? a.k : a.q) + unit * a.dim;
-            float* dst = (which ? a.ck : a.cq) + (int64_t)t * a.ld + unit * a.dim;
-            float x[4], ss = 0.f;
+        for (int r = 0; r < kConvRows; r++) ss[r] = 0.f;
 #pragma unroll
-            for (int i = 0; i < 4; i++) {
-                const int d = lane + 64 * i;
-                x[i] = d < a.dim ? conv_row(a, src + d, which * qk + unit * a.dim + d, t) : 0.f;
-                ss = fmaf(x[i], x[i], ss);
-            }
-            const float f = (which ? 1.0f : 1.0f / sqrtf((float)a.dim)) / sqrtf(wave_sum(ss) + kUnitEps);
+        for (int i = 0; i < 4; i++) {
+            const int d = lane + 64 * i;
+            if (64 * i >= a.dim) break;
+            conv_rows(a, src + min(d, a.dim - 1), which * qk + head * a.dim + min(d, a.dim - 1), t0, y[i]);
+#pragma unroll
+            for (int r = 0; r < kConvRows; r++) ss[r] = d < a.dim ? fmaf(y[i][r], y[i][r], ss[r]) : ss[r];
+        }
+#pragma unroll
+        for (int r = 0; r < kConvRows; r++) {
+            const float f = (which ? 1.0f : 1.0f / sqrtf((float)a.dim)) / sqrtf(wave_sum(ss[r]) + kUnitEps);
 #pragma unroll
             for (int i = 0; i < 4; i++)
-                if (lane + 64 * i < a.dim) dst[lane + 64 * i] = x[i] * f;
+                if (lane + 64 * i < a.dim && r < rows) dst[(int64_t)r * a.ld + lane + 64 * i] = y[i][r] * f;
         }
         return;
     }
+    const int c = (unit - 2 * a.kv_heads) * 64 + lane;
+    if (c >= a.vcols) return;
+    conv_rows(a, a.v + c, 2 * qk + c, t0, y[0]);
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-        const int c = (unit - a.kv_heads) * 256 + 64 * i + lane;
-        if (c < a.vcols) a.cv[(int64_t)t * a.ld + c] = conv_row(a, a.v + c, 2 * qk + c, t);
-    }
+    for (int r = 0; r < kConvRows; r++)
+        if (r < rows) a.cv[(int64_t)(t0 + r) * a.ld + c] = y[0][r];
 }
 
 // the last tokens' inputs to the ring (after every row has read what was there); grid (channels / 256, tokens kept)
@@ -126,74 +148,75 @@ __device__ __forceinline__ void level_factors(const float (&gl)[kChunk], float (
 template <int DP>
 __global__ __launch_bounds__(64) void gated_chunk_kernel(const ChunkArgs p) {
     constexpr int kPitch = DP + 4, kSets = (DP + 63) / 64, kTiles = DP / 16;
-    __shared__ __align__(16) float raw[3][kChunk * kPitch];  // q, k, log2 of the factors
-    __shared__ __align__(16) float op[2][kChunk * kPitch];   // a level's q and k; then K0 and R0
-    __shared__ __align__(16) float tri[2][kChunk][20];       // L, G
+    __shared__ __align__(16) float op[2][kChunk * kPitch];  // a level's q and k; then K0 and R0
+    __shared__ __align__(16) float tri[2][kChunk][20];      // L, G
     const int lane = threadIdx.x, chunk = blockIdx.x, h = blockIdx.y, t0 = chunk * kChunk, t16 = lane & 15, q4 = lane >> 4;
     const int kvh = h / p.per_kv, dim = p.dim, last = p.n - 1;
     float* out = p.ops + ((int64_t)h * gridDim.x + chunk) * chunk_floats(DP, p.vdim);
     const float rate = p.rate[h];
-    float beta[kChunk];
+    float beta[kChunk], q[kSets][kChunk], k[kSets][kChunk], gl[kSets][kChunk];  // this lane's channels; gl: log2 of the factors
 #pragma unroll
     for (int t = 0; t < kChunk; t++) beta[t] = t0 + t < p.n ? p.beta[(int64_t)min(t0 + t, last) * p.ld + h] : 0.f;
-#pragma unroll 1
+#pragma unroll
     for (int i = 0; i < kSets; i++) {
-        const int d = lane + 64 * i;
-        if (d >= DP) continue;
+        const int d = lane + 64 * i, dd = min(d, dim - 1);
+#pragma unroll
+        for (int t = 0; t < kChunk; t++) {
+            const int64_t row = (int64_t)min(t0 + t, last) * p.ld;
+            q[i][t] = p.q[row + kvh * dim + dd];
+            k[i][t] = p.k[row + kvh * dim + dd];
+            gl[i][t] = p.z[row + h * dim + dd];
+        }
 #pragma unroll
         for (int t = 0; t < kChunk; t++) {
             const bool in = d < dim && t0 + t < p.n;
-            const int64_t row = (int64_t)min(t0 + t, last) * p.ld;
-            const int dd = min(d, dim - 1);
-            raw[0][t * kPitch + d] = in ? p.q[row + kvh * dim + dd] : 0.f;
-            raw[1][t * kPitch + d] = in ? p.k[row + kvh * dim + dd] : 0.f;
-            raw[2][t * kPitch + d] = in ? log2_factor(p.z[row + h * dim + dd], rate) : 0.f;
+            q[i][t] = in ? q[i][t] : 0.f;
+            k[i][t] = in ? k[i][t] : 0.f;
+            gl[i][t] = in ? log2_factor(gl[i][t], rate) : 0.f;
         }
     }
-    __syncthreads();
     // the triangles, level by level; level 0: the diagonal of G
     f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = kk;
-    auto multiply = [&](const float* q, const float* k, int b) __attribute__((always_inline)) {
-        f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = x;
+    auto level = [&](auto width) __attribute__((always_inline)) {
+        constexpr int B = decltype(width)::value;
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < kSets; i++) {
+            const int d = lane + 64 * i;
+            if (d >= DP) continue;
+            float f[kChunk];
+#pragma unroll
+            for (int t = 0; t < kChunk; t++) f[t] = 1.f;
+            if constexpr (B > 0) level_factors<B>(gl[i], f);
+#pragma unroll
+            for (int t = 0; t < kChunk; t++) {
+                op[0][t * kPitch + d] = q[i][t] * f[t];
+                op[1][t * kPitch + d] = k[i][t] * f[t];
+            }
+        }
+        __syncthreads();
+        f32x4 x[2], y[2];
+#pragma unroll
+        for (int i = 0; i < 2; i++) x[i] = y[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll 2
         for (int c = 0; c < kTiles; c++) {
             const int at = t16 * kPitch + 16 * c + 4 * q4;
-            const f32x4 qv = load4(q + at), kv = load4(k + at);
+            const f32x4 qv = load4(&op[0][at]), kv = load4(&op[1][at]);
 #pragma unroll
             for (int e = 0; e < 4; e++) {
-                x = mma(kv[e], kv[e], x);
-                y = mma(qv[e], kv[e], y);
+                if constexpr (B > 0) x[e & 1] = mma(kv[e], kv[e], x[e & 1]);
+                y[e & 1] = mma(qv[e], kv[e], y[e & 1]);
             }
         }
 #pragma unroll
         for (int e = 0; e < 4; e++) {
             const int t = 4 * q4 + e, s = t16, diff = t ^ s;
-            const bool mine = b == 0 ? diff == 0 : t > s && diff >= b && diff < 2 * b;
-            kk[e] = mine ? x[e] : kk[e];
-            qk[e] = mine ? y[e] : qk[e];
+            const bool mine = B == 0 ? diff == 0 : t > s && diff >= B && diff < 2 * B;
+            kk[e] = mine ? x[0][e] + x[1][e] : kk[e];
+            qk[e] = mine ? y[0][e] + y[1][e] : qk[e];
         }
     };
-    multiply(raw[0], raw[1], 0);
-    auto level = [&](auto width) __attribute__((always_inline)) {
-        constexpr int B = decltype(width)::value;
-#pragma unroll 1
-        for (int i = 0; i < kSets; i++) {
-            const int d = lane + 64 * i;
-            if (d >= DP) continue;
-            float gl[kChunk], f[kChunk];
-#pragma unroll
-            for (int t = 0; t < kChunk; t++) gl[t] = raw[2][t * kPitch + d];
-            level_factors<B>(gl, f);
-#pragma unroll
-            for (int t = 0; t < kChunk; t++) {
-                op[0][t * kPitch + d] = raw[0][t * kPitch + d] * f[t];
-                op[1][t * kPitch + d] = raw[1][t * kPitch + d] * f[t];
-            }
-        }
-        __syncthreads();
-        multiply(op[0], op[1], B);
-        __syncthreads();
-    };
+    level(std::integral_constant<int, 0>());
     level(std::integral_constant<int, 8>());
     level(std::integral_constant<int, 4>());
     level(std::integral_constant<int, 2>());
@@ -214,18 +237,17 @@ __global__ __launch_bounds__(64) void gated_chunk_kernel(const ChunkArgs p) {
             x[t] *= beta[t];
         }
     };
-#pragma unroll 1
+#pragma unroll
     for (int i = 0; i < kSets; i++) {
         const int d = lane + 64 * i;
         if (d >= DP) continue;
-        float gl[kChunk], x[kChunk], upto = 0.f;
+        float x[kChunk], upto = 0.f;
 #pragma unroll
         for (int t = 0; t < kChunk; t++) {
-            gl[t] = raw[2][t * kPitch + d];
-            upto += gl[t];
+            upto += gl[i][t];
             const float f = __builtin_amdgcn_exp2f(upto);
-            x[t] = raw[1][t * kPitch + d] * f;
-            op[1][t * kPitch + d] = raw[0][t * kPitch + d] * f;
+            x[t] = k[i][t] * f;
+            op[1][t * kPitch + d] = q[i][t] * f;
         }
         out[off_w(DP) + d] = __builtin_amdgcn_exp2f(upto);
         solve(x);
@@ -234,8 +256,8 @@ __global__ __launch_bounds__(64) void gated_chunk_kernel(const ChunkArgs p) {
         float after = 0.f;
 #pragma unroll
         for (int t = kChunk - 1; t >= 0; t--) {
-            x[t] = raw[1][t * kPitch + d] * __builtin_amdgcn_exp2f(after);
-            after += gl[t];
+            x[t] = k[i][t] * __builtin_amdgcn_exp2f(after);
+            after += gl[i][t];
         }
         float* frag = out + off_kt(DP) + ((d >> 4) * 64 + (d & 15)) * 4;  // tile d / 16, lane 16 q + d % 16
 #pragma unroll
@@ -360,15 +382,24 @@ struct StepArgs {
     float* state;
 };
 
-// row . t, shared by eight lanes; the total in all of them
+// row . t over rank_pad columns (zeros of the row from its rank on), shared by eight lanes; the total in all of them
 template <typename W>
-__device__ __forceinline__ float low_rank_dot(const W* row, const float* t, int rank, int l) {
+__device__ __forceinline__ float low_rank_dot(const W* row, const float* t, int rank_pad, int l) {
     float z = 0.f;
-    for (int i = l; i < rank; i += 8) {
-        float f;
-        if constexpr (sizeof(W) == 2) f = __uint_as_float((uint32_t)row[i] << 16);
-        else f = row[i];
-        z = fmaf(f, t[i], z);
+#pragma unroll 2
+    for (int i = 8 * l; i < rank_pad; i += 64) {
+        float f[8];
+        const float4 a = *reinterpret_cast<const float4*>(t + i), b = *reinterpret_cast<const float4*>(t + i + 4);
+        if constexpr (sizeof(W) == 2) {
+            const uint4 w = *reinterpret_cast<const uint4*>(row + i);
+            const uint32_t u[4] = {w.x, w.y, w.z, w.w};
+#pragma unroll
+            for (int j = 0; j < 4; j++) f[2 * j] = __uint_as_float(u[j] << 16), f[2 * j + 1] = __uint_as_float(u[j] & 0xFFFF0000u);
+        } else {
+            const float4 c = *reinterpret_cast<const float4*>(row + i), d = *reinterpret_cast<const float4*>(row + i + 4);
+            f[0] = c.x, f[1] = c.y, f[2] = c.z, f[3] = c.w, f[4] = d.x, f[5] = d.y, f[6] = d.z, f[7] = d.w;
+        }
+        z += ((f[0] * a.x + f[1] * a.y) + (f[2] * a.z + f[3] * a.w)) + ((f[4] * b.x + f[5] * b.y) + (f[6] * b.z + f[7] * b.w));
     }
     return lane_group_sum<8>(z);
 }
@@ -394,10 +425,10 @@ __global__ __launch_bounds__(64 * NW) void gated_step_kernel(const StepArgs a) {
     for (int r = tid >> 3; r < DP + vdim; r += kThreads / 8) {
         const int d = r - DP, l = tid & 7;
         if (r < DP) {
-            const float z = low_rank_dot((const W*)p.w_a + (int64_t)(h * dim + min(r, dim - 1)) * p.rank_a_pad, p.a_low, p.rank_a, l);
+            const float z = low_rank_dot((const W*)p.w_a + (int64_t)(h * dim + min(r, dim - 1)) * p.rank_a_pad, p.a_low, p.rank_a_pad, l);
             if (l == 0) vec[2][r] = r < dim ? __builtin_amdgcn_exp2f(log2_factor(z + p.bias_a[h * dim + r], a.rate[h])) : 0.f;
         } else {
-            const float z = low_rank_dot((const W*)p.w_g + (int64_t)(h * vdim + d) * p.rank_g_pad, p.g_low, p.rank_g, l);
+            const float z = low_rank_dot((const W*)p.w_g + (int64_t)(h * vdim + d) * p.rank_g_pad, p.g_low, p.rank_g_pad, l);
             if (l == 0) sg[d] = skn_sigmoid(z);
         }
     }
@@ -490,8 +521,8 @@ int skn_gated_delta_rows(skn_ctx* ctx, skn_rstate* st, int seq, const skn_channe
     SKN_REQUIRE(ctx, st->taps > 0, SKN_ERR_STATE, "gated delta rule: the state has no convolutions");
     SKN_REQUIRE(ctx, n > 0 && st->heads <= 65535, SKN_ERR_SHAPE, "gated delta rule: %d tokens x %d heads", n, st->heads);
     ConvArgs c = {q, k, v, ld, n, pos0, st->seq_conv(seq), p.conv, st->taps, st->kv_heads, st->dim, st->heads * st->vdim, st->channels, cq, ck, cv};
-    const int units = st->kv_heads + (c.vcols + 255) / 256;
-    skn_launch(ctx, conv_rows_kernel, dim3(n, (units + 3) / 4), dim3(256), 0, c);
+    const int units = 2 * st->kv_heads + (c.vcols + 63) / 64;
+    skn_launch(ctx, conv_rows_kernel, dim3((n + kConvRows - 1) / kConvRows, (units + 3) / 4), dim3(256), 0, c);
     SKN_LAUNCH_CHECK(ctx);
     skn_launch(ctx, conv_keep_kernel, dim3((st->channels + 255) / 256, std::min(n, st->taps)), dim3(256), 0, c, st->seq_conv(seq));
     SKN_LAUNCH_CHECK(ctx);

@@ -243,8 +243,7 @@ int mixer_step(skn_ctx* ctx, skn_hybrid* m, Layer& L, int max_ctx, skn_matvec_sr
             d.a_low = m->rank, d.g_low = m->rank2;
             d.w_a = L.decay.w, d.w_g = L.gate.w;
             d.w_type = L.decay.type;
-            d.rank_a = L.p.rank, d.rank_a_pad = L.decay.k_pad;
-            d.rank_g = L.p.rank_gate, d.rank_g_pad = L.gate.k_pad;
+            d.rank_a_pad = L.decay.k_pad, d.rank_g_pad = L.gate.k_pad;
             d.bias_a = L.decay.bias;
             d.norm = L.p.o_norm;
             d.eps = m->cfg.norm_eps;

@@ -51,9 +51,9 @@ int skn_gated_delta_rows(skn_ctx* ctx, skn_rstate* st, int seq, const skn_channe
 // norm and gate.  beta: after its sigmoid.
 struct skn_gated_step {
     const float *q, *k, *v, *beta;
-    const float *a_low, *g_low;  // [rank_a], [rank_g]
+    const float *a_low, *g_low;  // [rank_a_pad], [rank_g_pad]: finite beyond the ranks
     const void *w_a, *w_g;       // [heads * dim][rank_a_pad], [heads * vdim][rank_g_pad] of w_type
-    int w_type, rank_a, rank_a_pad, rank_g, rank_g_pad;
+    int w_type, rank_a_pad, rank_g_pad;
     const float* bias_a;  // [heads * dim]
     const float* norm;    // [heads * vdim]
     float eps;

@@ -60,7 +60,7 @@ def test_logits_do_not_depend_on_the_cut(hip, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("tile", [1, 2, 3, 4])
+@pytest.mark.parametrize("tile", [1, 2, 3, 4, 5])
 def test_every_tile_of_the_gemm(hip, tile, dtype):
     cfg, *ranks = cases.MODELS["mixed"]
     w = cases.weights(cfg, *ranks)
