@@ -10,6 +10,8 @@
 // tiles w, w + 4, ... up to the causal limit with the online softmax, and the four partial results are merged
 // through LDS: S^T = K Q^T (scores of a query sit in one lane column: its maximum and sum need no
 // cross-lane traffic beyond the two lane halves), P = exp2(S - max), O^T += V^T P^T.
+// A query may see a range of the keys only (a window, or its chunk): tiles outside the range of a block of queries are neither copied
+// nor visited.  Latents come expanded: attn_frag_rows_kernel takes their keys and values row by row.
 // Precision: K and V are the cached fp16 values; q (pre-multiplied by scale * log2 e) and P enter as fp16 pairs
 // hi + lo (two matrix instructions per step), products and sums are fp32.
 #include "kv.h"

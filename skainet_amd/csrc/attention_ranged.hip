@@ -21,39 +21,37 @@ __global__ __launch_bounds__(256) void ranged_prep_kernel(const skn_ranged_attn 
     if (tid < half) skn_rope_sincos_freq(pos, p.rot_freq[tid], &sn[tid], &cs[tid]);
     const int page = table[pos / page_tokens], slot = pos % page_tokens, heads = p.n_head + kv_heads;
     __syncthreads();
-    for (int base = 0; base < heads; base += 4) {  // (all wavefronts take every turn: the barriers are theirs together)
-        const int h = base + wave;
+    for (int h = wave; h < heads; h += 4) {
         const bool is_q = h < p.n_head;
         const float* src = is_q ? q + (int64_t)row * ldq + h * kdim : k + (int64_t)row * ldk + (h - p.n_head) * kdim;
         const float* norm = is_q ? p.q_norm : p.k_norm;
-        if (h < heads) {
-            float r[4], ss = 0.f;
+        float r[4], ss = 0.f;
 #pragma unroll
-            for (int j = 0; j < 4; j++) {
-                const int e = lane + 64 * j;
-                r[j] = e < kdim ? src[e] : 0.f;
-                ss = fmaf(r[j], r[j], ss);
-            }
-            const float f = norm ? 1.0f / sqrtf(wave_sum(ss) / (float)kdim + p.eps) : 1.f;
-#pragma unroll
-            for (int j = 0; j < 4; j++) {
-                const int e = lane + 64 * j;
-                x[wave][e] = r[j] * f * (norm && e < kdim ? norm[e] : 1.f);
-            }
+        for (int j = 0; j < 4; j++) {
+            const int e = lane + 64 * j;
+            r[j] = e < kdim ? src[e] : 0.f;
+            ss = fmaf(r[j], r[j], ss);
         }
-        __syncthreads();
-        if (h < heads) {
+        const float f = norm ? 1.0f / sqrtf(wave_sum(ss) / (float)kdim + p.eps) : 1.f;
 #pragma unroll
-            for (int j = 0; j < 4; j++) {
-                const int e = lane + 64 * j;
-                float y = x[wave][e];
-                if (e < half) y = y * cs[e] - x[wave][e + half] * sn[e];
-                else if (e < p.rot_dims) y = y * cs[e - half] + x[wave][e - half] * sn[e - half];
-                if (is_q && e < width) q_prep[((int64_t)row * p.n_head + h) * width + e] = y;
-                else if (!is_q && e < kdim) store_cached(k_pool + (((int64_t)page * kv_heads + (h - p.n_head)) * page_tokens + slot) * width + e, y);
-            }
+        for (int j = 0; j < 4; j++) {
+            const int e = lane + 64 * j;
+            x[wave][e] = r[j] * f * (norm && e < kdim ? norm[e] : 1.f);
         }
-        __syncthreads();
+        // (a wavefront's own part of LDS, whose accesses take effect in order)
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+#pragma unroll
+        for (int j = 0; j < 4; j++) {
+            const int e = lane + 64 * j;
+            float y = x[wave][e];
+            if (e < half) y = y * cs[e] - x[wave][e + half] * sn[e];
+            else if (e < p.rot_dims) y = y * cs[e - half] + x[wave][e - half] * sn[e - half];
+            if (is_q && e < width) q_prep[((int64_t)row * p.n_head + h) * width + e] = y;
+            else if (!is_q && e < kdim) store_cached(k_pool + (((int64_t)page * kv_heads + (h - p.n_head)) * page_tokens + slot) * width + e, y);
+        }
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+        __builtin_amdgcn_wave_barrier();
     }
     for (int e = tid; e < kv_heads * vdim; e += 256) {
         const int h = e / vdim, d = e - h * vdim;
